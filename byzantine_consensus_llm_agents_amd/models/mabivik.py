@@ -253,9 +253,9 @@ class MabivikModel:
                 L["q_norm"], L["uq"], L["o"] = f32(q + "dq.norm"), get(q + "uq"), get(q + "o")
                 if m.kv_from < 0:
                     L["kv_norm"] = f32(q + "dkv.norm")
-                # per head: W_uk[h]^T as the weight of a linear (kv_rank outputs from dim inputs), W_uv[h]
-                L["uk_t"] = get(q + "uk").reshape(m.heads, m.dim, m.kv_rank).transpose(1, 2).contiguous()
-                L["uv"] = get(q + "uv").reshape(m.heads, m.vdim, m.kv_rank).contiguous()
+                # per head, as right operands [inputs, outputs]: W_uk[h] (dim -> kv_rank), W_uv[h]^T (kv_rank -> vdim)
+                L["uk"] = get(q + "uk").reshape(m.heads, m.dim, m.kv_rank).contiguous()
+                L["uv_t"] = get(q + "uv").reshape(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous()
                 L["inv_freq"], L["amp"] = ramp_inv_freq(m.rot_dims, m.rot_base, m.rot_scaling, dev)
             elif l.type == "delta":
                 names = (q + "q", q + "k", q + "v")
@@ -306,13 +306,13 @@ class MabivikModel:
             off_g += m.key_width
         q = ops.linear(ops.rmsnorm_cols(y, 0, m.q_rank, L["q_norm"], eps, self.dtype), L["uq"]).view(T, m.heads, m.dim + m.rot_dim)
         qf = torch.empty(T, m.heads, m.key_width, dtype=self.dtype, device=h.device)
-        ops.head_linear(q[:, :, :m.dim], L["uk_t"], qf[:, :, :m.kv_rank])
+        ops.head_linear(q[:, :, :m.dim], L["uk"], qf[:, :, :m.kv_rank])
         ops.rope_half_tail(q, m.dim, qf, m.kv_rank, meta.positions, L["inv_freq"], L["amp"])
         lat = ops.multimap_attention(qf, k_cache, v_cache, meta, m.scale, 1, 0.0, -1.0, 1.0, m.kv_rank, m.window, None)
         gate = y[:, off_g:off_g + m.heads * m.vdim]
         if sel is not None:
             lat, gate = lat.index_select(0, sel), gate.index_select(0, sel)
-        att = ops.head_linear(lat.view(-1, m.heads, m.kv_rank), L["uv"])
+        att = ops.head_linear(lat.view(-1, m.heads, m.kv_rank), L["uv_t"])
         return ops.linear(ops.gate_mul(att.view(-1, m.heads * m.vdim), gate, "sigmoid"), L["o"])
 
     def _delta(self, m, L, S, h, meta, sel):

@@ -855,11 +855,11 @@ def rope_half_tail(src, src_off: int, dst, dst_off: int, positions, inv_freq, am
 
 
 def head_linear(x3, w, out3=None):
-    """``out3[t, h] = w[h] x3[t, h]``: x3 [T, H, K] (any strides with a unit last one), w [H, N, K],
-    out3 [T, H, N] (a view to fill, or None: a new contiguous tensor)."""
+    """``out3[t, h] = x3[t, h] w[h]``: x3 [T, H, K] (any strides with a unit last one), w [H, K, N]
+    contiguous, out3 [T, H, N] (a view to fill, or None: a new contiguous tensor)."""
     if out3 is None:
-        out3 = torch.empty(x3.shape[0], x3.shape[1], w.shape[1], dtype=x3.dtype, device=x3.device)
-    torch.bmm(x3.transpose(0, 1), w.transpose(1, 2), out=out3.transpose(0, 1))
+        out3 = torch.empty(x3.shape[0], x3.shape[1], w.shape[2], dtype=x3.dtype, device=x3.device)
+    torch.bmm(x3.transpose(0, 1), w, out=out3.transpose(0, 1))
     return out3
 
 

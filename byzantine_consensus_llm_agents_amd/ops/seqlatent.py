@@ -97,15 +97,17 @@ def seqlatent_ops(lib):
         return dst
 
     def head_linear(x3, w, out3=None):
-        """Per-head products on the vendor's batched GEMM (fp32 accumulation; true fp32 for fp32 operands)."""
-        _req(x3.dim() == 3 and w.dim() == 3 and x3.shape[1] == w.shape[0] and x3.shape[2] == w.shape[2] and x3.stride(2) == 1
-             and x3.dtype == w.dtype and w.is_contiguous(), "head_linear: x [T, H, K], w [H, N, K]")
+        """Per-head products on the vendor's batched GEMM (fp32 accumulation; true fp32 for fp32 operands).
+        The weight is the right operand as it lies, [H, K, N]: the batched bf16 product has faulted the
+        GPU with a transposed view there."""
+        _req(x3.dim() == 3 and w.dim() == 3 and x3.shape[1] == w.shape[0] and x3.shape[2] == w.shape[1] and x3.stride(2) == 1
+             and x3.dtype == w.dtype and w.is_contiguous(), "head_linear: x [T, H, K], w [H, K, N]")
         if out3 is None:
-            out3 = torch.empty(x3.shape[0], x3.shape[1], w.shape[1], dtype=x3.dtype, device=x3.device)
-        _req(out3.shape == (x3.shape[0], x3.shape[1], w.shape[1]) and out3.stride(2) == 1 and out3.dtype == x3.dtype,
+            out3 = torch.empty(x3.shape[0], x3.shape[1], w.shape[2], dtype=x3.dtype, device=x3.device)
+        _req(out3.shape == (x3.shape[0], x3.shape[1], w.shape[2]) and out3.stride(2) == 1 and out3.dtype == x3.dtype,
              "head_linear: out [T, H, N]")
         if x3.shape[0]:
-            torch.bmm(x3.transpose(0, 1), w.transpose(1, 2), out=out3.transpose(0, 1))
+            torch.bmm(x3.transpose(0, 1), w, out=out3.transpose(0, 1))
         return out3
 
     def gate_mul(x, gate, kind, group=1):
