@@ -47,14 +47,14 @@ import json
 import os
 import threading
 import time
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from typing import Deque, Dict, List, Optional
 
 import numpy as np
 import torch
 
 from ..bcg.config import ENGINE_CONFIG
-from ..models.config import ModelConfig, get_model_config
+from ..models.config import ARCHITECTURES, ModelConfig, get_model_config
 from ..models import build_model
 from ..models.transformer import AttnMeta, TPGroup
 from ..ops import get_ops
@@ -185,6 +185,8 @@ class InferenceEngine:
         self.prompt_lens: Dict[int, List[int]] = collections.defaultdict(list)
         self._carry: List["_Request"] = []  # admitted, prefill incomplete (pending), oldest first
         cfg = args.model_cfg
+        if getattr(cfg, "learned_positions", False):  # no position vector beyond the table: sequences end there
+            self.args = args = replace(args, max_model_len=min(args.max_model_len, cfg.max_position))
         self.backend = args.backend
         if self.backend == "hip" and not torch.cuda.is_available():
             raise RuntimeError("hip backend requested but no GPU is visible")
@@ -199,7 +201,7 @@ class InferenceEngine:
         self.ops = get_ops(self.backend)
 
         model_dir = args.weights if args.weights not in ("random", "auto") else None
-        if model_dir and not os.path.exists(os.path.join(model_dir, "tokenizer.json")) and cfg.family in ("mofidra", "padadra", "mabivik", "sitidra"):
+        if model_dir and not os.path.exists(os.path.join(model_dir, "tokenizer.json")) and cfg.family in ARCHITECTURES:
             from .tokenizer import IdTokenizer
             self.tokenizer = IdTokenizer(cfg.vocab_size)  # a checkpoint of weights only: prompts are token ids
         else:

@@ -14,6 +14,9 @@ def model_class(family: str):
     if family == "sitidra":
         from .sitidra import SitidraModel
         return SitidraModel
+    if family == "sadodra":
+        from .sadodra import SadodraModel
+        return SadodraModel
     from .transformer import DecoderModel
     return DecoderModel
 

@@ -383,11 +383,12 @@ class LatentAttentionSpec:
     """Softmax attention whose keys and values are read from one low-rank latent per token: the
     cache holds the RMS-normed latent ``c`` (``kv_rank``) and one rotated key part (``rot_dim``)
     shared by all heads; head h's unrotated key is ``W_uk[h] c`` (``dim``), its value ``W_uv[h] c``
-    (``vdim``).  Queries pass a latent of their own (``q_rank``).  Rotary (feature i pairs with
+    (``vdim``).  Queries pass a latent of their own (``q_rank``; 0: they come straight from the input).  Rotary (feature i pairs with
     i + rot_dims / 2) acts on the first ``rot_dims`` features of the rotated part; ``rot_scaling``
     = (factor, original, fast, slow) ramps the frequencies between two turn counts and multiplies
     cos and sin by ``0.1 ln(factor) + 1``.  ``window`` keys are visible (0 = all); ``kv_from``: the
-    layer whose cache this one reads instead of holding one (-1 = its own)."""
+    layer whose cache this one reads instead of holding one (-1 = its own); ``head_gate``: one sigmoid
+    output gate per head instead of one per value feature."""
     heads: int
     dim: int
     rot_dim: int
@@ -400,6 +401,7 @@ class LatentAttentionSpec:
     rot_base: float = 10000.0
     rot_scaling: Optional[tuple] = None
     kv_from: int = -1
+    head_gate: bool = False
 
     @property
     def q_width(self) -> int:
@@ -409,6 +411,10 @@ class LatentAttentionSpec:
     def key_width(self) -> int:
         """Cached key features per token: the latent and the shared rotated part."""
         return self.kv_rank + self.rot_dim
+
+    @property
+    def gate_width(self) -> int:
+        return self.heads if self.head_gate else self.heads * self.vdim
 
 
 @dataclass(frozen=True)
@@ -735,6 +741,136 @@ class SitidraConfig:
         return n
 
 
+@dataclass(frozen=True)
+class BiasedAttentionSpec:
+    """GQA softmax attention without rotation whose values are the keys as projected (``dim`` features
+    each): one RMS norm with weights over the whole q (and k) projection, a query temperature
+    ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` (``temp_every`` 0 = none), scaled scores capped by
+    ``softcap tanh(. / softcap)`` (0 = none), then a distance bias ``2^(-8 (h + 1) / heads) (i - j)`` taken
+    off, and a sliding window of ``window`` keys (0 = all)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    window: int = 0
+    softcap: float = 0.0
+    temp_coef: float = 0.0
+    temp_every: int = 0
+
+    @property
+    def q_width(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def k_width(self) -> int:
+        return self.kv_heads * self.dim
+
+
+@dataclass(frozen=True)
+class SadodraLayer:
+    type: str                    # "attention" | "latent_attention"
+    mixer: object                # BiasedAttentionSpec | LatentAttentionSpec
+    mlp: Optional[FeedForwardSpec]
+
+
+@dataclass(frozen=True)
+class SadodraConfig:
+    """Sadodra: ``x <- x + norm1(mixer(x))`` then ``x <- x + norm2(ff(x))`` with layer norms (weight and
+    bias) on the sublayers' outputs only, a learned position vector added to the embedding
+    (``max_position`` rows), mixers of two kinds (windowed attention with capped and distance-biased
+    scores, latent attention without positions) in the order the config lists, dense gated gelu
+    feed-forwards.  Everything is read from the model directory's config.json."""
+    name: str
+    hidden_size: int
+    vocab_size: int
+    layers: tuple
+    max_position: int
+    rms_eps: float = 1e-6
+    family: str = "sadodra"
+    tie_embeddings: bool = False
+    learned_positions: bool = True    # a sequence cannot be longer than max_position
+
+    @staticmethod
+    def _latent(m: dict, layers: list) -> LatentAttentionSpec:
+        spec = LatentAttentionSpec(
+            heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=0, vdim=int(m["vdim"]), q_rank=0, kv_rank=int(m["kv_rank"]),
+            scale=float(m["scale"]), window=int((m.get("mask") or {}).get("size", 0)),
+            kv_from=-1 if m.get("kv_from") is None else int(m["kv_from"]), head_gate=True)
+        if spec.kv_from >= 0:
+            src = layers[spec.kv_from].mixer if spec.kv_from < len(layers) else None
+            if not isinstance(src, LatentAttentionSpec) or src.kv_from >= 0 or src.kv_rank != spec.kv_rank:
+                raise ValueError("Sadodra: kv_from names an earlier latent-attention layer with a latent of its own, of the same size")
+        return spec
+
+    @classmethod
+    def from_dict(cls, c: dict, name: str = "sadodra") -> "SadodraConfig":
+        layers = []
+        for entry in c["layers"]:
+            m, kind = entry["mixer"], entry["type"]
+            if kind == "attention":
+                temp = m.get("q_temp") or {}
+                mixer = BiasedAttentionSpec(
+                    heads=int(m["heads"]), kv_heads=int(m.get("kv_heads") or m["heads"]), dim=int(m["dim"]),
+                    scale=float(m["scale"]), window=int((m.get("mask") or {}).get("size", 0)),
+                    softcap=float(m.get("softcap") or 0.0), temp_coef=float(temp.get("coef", 0.0)), temp_every=int(temp.get("every", 0)))
+                if mixer.heads % mixer.kv_heads or int(m.get("vdim", mixer.dim)) != mixer.dim:
+                    raise ValueError("Sadodra: heads must be a multiple of kv_heads, vdim equal to dim (the values are the keys)")
+                if mixer.window < 0 or mixer.softcap < 0 or (temp and mixer.temp_every < 1):
+                    raise ValueError("Sadodra: mask.size and softcap not negative, q_temp.every at least 1")
+            elif kind == "latent_attention":
+                mixer = cls._latent(m, layers)
+            else:
+                raise ValueError(f"Sadodra: unknown layer type {kind!r}")
+            f = entry.get("mlp")
+            if f is not None and f.get("kind", "dense") != "dense":
+                raise ValueError(f"Sadodra: unknown feed-forward kind {f['kind']!r}")
+            layers.append(SadodraLayer(kind, mixer, FeedForwardSpec("dense", int(f["ff"])) if f else None))
+        return cls(name=name, hidden_size=int(c["width"]), vocab_size=int(c["vocab"]), layers=tuple(layers),
+                   max_position=int(c["max_positions"]), rms_eps=float(c["norm"]["eps"]))
+
+    def to_dict(self) -> dict:
+        """The config.json form (inverse of `from_dict`)."""
+        out = []
+        for l in self.layers:
+            m = l.mixer
+            if l.type == "attention":
+                mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim, "vdim": m.dim, "scale": m.scale}
+                if m.softcap:
+                    mixer["softcap"] = m.softcap
+                if m.temp_every:
+                    mixer["q_temp"] = {"coef": m.temp_coef, "every": m.temp_every}
+            else:
+                mixer = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim, "kv_rank": m.kv_rank, "scale": m.scale}
+                if m.kv_from >= 0:
+                    mixer["kv_from"] = m.kv_from
+            if m.window:
+                mixer["mask"] = {"size": m.window}
+            out.append({"type": l.type, "mixer": mixer, "mlp": {"kind": "dense", "ff": l.mlp.ff} if l.mlp else None})
+        return {"architecture": "Sadodra", "width": self.hidden_size, "vocab": self.vocab_size,
+                "max_positions": self.max_position, "norm": {"eps": self.rms_eps}, "layers": out}
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def num_params(self) -> int:
+        W, n = self.hidden_size, (2 * self.vocab_size + self.max_position) * self.hidden_size
+        for l in self.layers:
+            m = l.mixer
+            if l.type == "attention":
+                n += W * (2 * m.q_width + m.k_width)
+            else:
+                n += W * (m.q_width + m.gate_width + m.heads * m.vdim) + m.heads * m.kv_rank * (m.dim + m.vdim)
+                n += W * m.key_width if m.kv_from < 0 else 0
+            n += 3 * W * l.mlp.ff if l.mlp is not None else 0
+        return n
+
+
+# config.json "architecture" (lower case) -> configuration class; these families take token ids
+# when a checkpoint ships no tokenizer
+ARCHITECTURES = {"mofidra": MofidraConfig, "padadra": PadadraConfig, "mabivik": MabivikConfig, "sitidra": SitidraConfig,
+                 "sadodra": SadodraConfig}
+
 PRESETS = {
     "Qwen/Qwen3-8B": ModelConfig("Qwen/Qwen3-8B", "qwen3", 4096, 36, 32, 8, 128, 12288, 151936,
                                  qk_norm=True, max_position=40960),
@@ -768,14 +904,9 @@ ALIASES = {
 def from_hf_config(path: str, name: Optional[str] = None):
     with open(os.path.join(path, "config.json")) as fh:
         c = json.load(fh)
-    if str(c.get("architecture", "")).lower() == "mofidra":
-        return MofidraConfig.from_dict(c, name or path)
-    if str(c.get("architecture", "")).lower() == "padadra":
-        return PadadraConfig.from_dict(c, name or path)
-    if str(c.get("architecture", "")).lower() == "mabivik":
-        return MabivikConfig.from_dict(c, name or path)
-    if str(c.get("architecture", "")).lower() == "sitidra":
-        return SitidraConfig.from_dict(c, name or path)
+    cls = ARCHITECTURES.get(str(c.get("architecture", "")).lower())
+    if cls is not None:
+        return cls.from_dict(c, name or path)
     arch = (c.get("model_type") or "").lower()
     family = "qwen3" if arch == "qwen3" else ("qwen2" if arch == "qwen2" else "mistral")
     heads = c["num_attention_heads"]

@@ -48,6 +48,7 @@ from typing import Dict, List, Optional
 import torch
 
 from .config import MabivikConfig
+from .latent import latent_mixer, latent_shapes, latent_weights
 from .transformer import AttnMeta, TPGroup
 
 
@@ -164,11 +165,7 @@ class MabivikModel:
             norm(p + "norm1")
             norm(p + "norm1b")
             if l.type == "latent_attention":
-                out.update({q + "dq": (m.q_rank, W), q + "dq.norm": (m.q_rank,), q + "uq": (m.q_width, m.q_rank),
-                            q + "uk": (m.heads * m.dim, m.kv_rank), q + "uv": (m.heads * m.vdim, m.kv_rank),
-                            q + "g": (m.heads * m.vdim, W), q + "o": (W, m.heads * m.vdim)})
-                if m.kv_from < 0:
-                    out.update({q + "dkv": (m.key_width, W), q + "dkv.norm": (m.kv_rank,)})
+                out.update(latent_shapes(m, W, q))
             elif l.type == "delta":
                 for n, width in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
                     out[q + n] = (width, W)
@@ -231,7 +228,6 @@ class MabivikModel:
         input are stacked into one GEMM weight, the per-head expansions into [H, ...] batches, every
         expert's gate and up rows into one [E, 2 ff, W] tensor."""
         c, dev, dt = self.cfg, self.device, self.dtype
-        from ..ops.reference import ramp_inv_freq
 
         def get(name, dtype=None):
             return sd[name].to(device=dev, dtype=dtype or dt).contiguous()
@@ -248,15 +244,7 @@ class MabivikModel:
             p, m, q = f"l{i}.", l.mixer, f"l{i}.mix."
             L = {"pre1": norm(p + "norm1"), "post1": norm(p + "norm1b")}
             if l.type == "latent_attention":
-                parts = [get(q + "dq")] + ([get(q + "dkv")] if m.kv_from < 0 else []) + [get(q + "g")]
-                L["fused"] = torch.cat(parts).contiguous()
-                L["q_norm"], L["uq"], L["o"] = f32(q + "dq.norm"), get(q + "uq"), get(q + "o")
-                if m.kv_from < 0:
-                    L["kv_norm"] = f32(q + "dkv.norm")
-                # per head, as right operands [inputs, outputs]: W_uk[h] (dim -> kv_rank), W_uv[h]^T (kv_rank -> vdim)
-                L["uk"] = get(q + "uk").reshape(m.heads, m.dim, m.kv_rank).contiguous()
-                L["uv_t"] = get(q + "uv").reshape(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous()
-                L["inv_freq"], L["amp"] = ramp_inv_freq(m.rot_dims, m.rot_base, m.rot_scaling, dev)
+                L.update(latent_weights(m, q, get, f32, dev))
             elif l.type == "delta":
                 names = (q + "q", q + "k", q + "v")
                 L["fused"] = torch.cat([get(n) for n in names] + [get(q + "b"), get(q + "a"), get(q + "g")]).contiguous()
@@ -297,23 +285,7 @@ class MabivikModel:
 
     # ------------------------------------------------------------- mixers
     def _latent_attention(self, m, L, h, meta, k_cache, v_cache, sel):
-        ops, eps, T = self.ops, self.cfg.rms_eps, h.shape[0]
-        y = ops.linear(h, L["fused"])
-        off_g = m.q_rank
-        if m.kv_from < 0:
-            ops.latent_kv_write(y, m.q_rank, m.kv_rank, m.rot_dim, L["kv_norm"], eps, meta.positions, meta.slots,
-                                L["inv_freq"], L["amp"], k_cache, v_cache)
-            off_g += m.key_width
-        q = ops.linear(ops.rmsnorm_cols(y, 0, m.q_rank, L["q_norm"], eps, self.dtype), L["uq"]).view(T, m.heads, m.dim + m.rot_dim)
-        qf = torch.empty(T, m.heads, m.key_width, dtype=self.dtype, device=h.device)
-        ops.head_linear(q[:, :, :m.dim], L["uk"], qf[:, :, :m.kv_rank])
-        ops.rope_half_tail(q, m.dim, qf, m.kv_rank, meta.positions, L["inv_freq"], L["amp"])
-        lat = ops.multimap_attention(qf, k_cache, v_cache, meta, m.scale, 1, 0.0, -1.0, 1.0, m.kv_rank, m.window, None)
-        gate = y[:, off_g:off_g + m.heads * m.vdim]
-        if sel is not None:
-            lat, gate = lat.index_select(0, sel), gate.index_select(0, sel)
-        att = ops.head_linear(lat.view(-1, m.heads, m.kv_rank), L["uv_t"])
-        return ops.linear(ops.gate_mul(att.view(-1, m.heads * m.vdim), gate, "sigmoid"), L["o"])
+        return latent_mixer(self.ops, m, L, h, meta, k_cache, v_cache, sel, self.cfg.rms_eps)
 
     def _delta(self, m, L, S, h, meta, sel):
         ops, eps = self.ops, self.cfg.rms_eps

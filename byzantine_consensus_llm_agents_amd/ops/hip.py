@@ -102,7 +102,12 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_multimap_split_keys": [],
         "bcg_multimap_attention": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                                    c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                   c_float, c_float, c_float, c_float, c_int, c_int, c_int, c_int, c_void_p, c_void_p],
+                                   c_float, c_float, c_float, c_float, c_int, c_int, c_int, c_int, c_void_p, c_float,
+                                   c_void_p, c_void_p],
+        "bcg_embed_position": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                               c_int, c_void_p],
+        "bcg_residual_layer_norm": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_void_p,
+                                    c_float, c_void_p, c_int, c_int, c_int, c_void_p],
         "bcg_embed_hashed_bigram": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
                                     c_void_p, c_int, c_int, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_void_p,
                                     c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -111,8 +116,8 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_short_conv": [c_void_p, c_int64, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                            c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
         "bcg_rope_pairs_kv_write": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int,
-                                    c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                    c_int, c_void_p],
+                                    c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                    c_float, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_rotate_pairs": [c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_hgrn2_prepare": [c_void_p, c_int64, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                               c_int, c_int, c_void_p],
@@ -145,7 +150,7 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_rope_half_tail": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_int,
                                c_int, c_int, c_void_p],
         "bcg_gate_mul": [c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p],
-        "bcg_gated_act": [c_void_p, c_void_p, c_int64, c_int, c_int, c_void_p],
+        "bcg_gated_act": [c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p],
         "bcg_ssm_prepare": [c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_gated_group_norm": [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_float, c_void_p,

@@ -406,14 +406,15 @@ def rope_multi_kv_write(qkv, positions, slots, n_q: int, n_kv: int, maps: int, d
 
 def multimap_attention(q, k_cache, v_cache, block_tables, q_start, seq_lens, scale: float, maps: int,
                        lam: float, head_eps: float, out_scale: float, vdim: int, window: int = 0, sink=None,
-                       chunk: int = 0):
+                       chunk: int = 0, softcap: float = 0.0, slopes=None):
     """Causal GQA attention with ``maps`` softmax maps per head over shared values:
     ``o = a_0 - lam * a_1`` (maps = 2; maps = 1: ``a_0``), then per head
     ``o / sqrt(mean(o^2) + head_eps) * out_scale`` (``head_eps < 0``: only the scale).
     Sequence b's query rows ``q_start[b]:q_start[b+1]`` are its last positions.  ``window`` > 0:
     position i sees only j with i - j < window.  ``chunk`` > 0: position i sees only j of its own
     chunk, floor(j / chunk) = floor(i / chunk), chunks counted from position 0.  ``sink`` fp32 [n_q]: the softmax denominator of
-    head h also holds ``exp(sink[h])`` (no key, no value, not scaled).  Returns
+    head h also holds ``exp(sink[h])`` (no key, no value, not scaled).  ``softcap`` > 0: the scaled score s
+    becomes ``softcap tanh(s / softcap)``; ``slopes`` fp32 [n_q]: then ``slopes[h] (i - j)`` is taken off.  Returns
     ``[T, n_q * vdim]``; fp32 math."""
     T, n_q, qd = q.shape
     dim = qd // maps
@@ -442,6 +443,10 @@ def multimap_attention(q, k_cache, v_cache, block_tables, q_start, seq_lens, sca
         o = None
         for m in range(maps):
             sc = torch.matmul(qb[..., m * dim:(m + 1) * dim], k[..., m * dim:(m + 1) * dim].transpose(1, 2)) * scale
+            if softcap > 0:
+                sc = softcap * torch.tanh(sc / softcap)
+            if slopes is not None:
+                sc = sc - slopes.float()[:, None, None] * (qpos - kpos).float()
             sc = sc.masked_fill(hidden, float("-inf"))
             if sink is not None:
                 col = sink.float()[:, None, None].expand(n_q, e - s, 1)
@@ -627,22 +632,33 @@ def _turn_pairs(x, ang):
     return torch.stack([a * c - b * s, b * c + a * s], dim=-1).flatten(-2)
 
 
+def query_temperature(positions, coef: float, every: int):
+    """fp32 [T]: ``1 + coef ln(floor((p + 1) / every) + 1)``."""
+    steps = torch.div(positions.long() + 1, int(every), rounding_mode="floor")
+    return 1.0 + float(coef) * torch.log(steps.float() + 1.0)
+
+
 def rope_pairs_kv_write(qkv, positions, slots, n_q: int, n_kv: int, dim: int, vdim: int, q_norm, k_norm, eps: float,
-                        inv_freq, v_inv_freq, k_cache, v_cache):
+                        inv_freq, v_inv_freq, k_cache, v_cache, v_is_k: bool = False, q_temp=None):
     """Row ``[q | k | v | ...]``: one RMS norm over the whole q part (weight ``q_norm``
     [n_q dim]; None = no norm) and one over the whole k part, then every q / k head's features
     (2i, 2i + 1), i < len(inv_freq), are turned by ``position * inv_freq[i]``; every v head's pairs
-    by ``position * v_inv_freq[i]`` (None: values as they are).  K / V go to the paged cache of
+    by ``position * v_inv_freq[i]`` (None: values as they are).  ``v_is_k``: the row is ``[q | k | ...]`` and the
+    values are the k part as projected, before its norm.  ``q_temp`` = (coef, every): q at position p is
+    multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)``.  K / V go to the paged cache of
     `rope_multi_kv_write`; returns q [T, n_q, dim]."""
     T = qkv.shape[0]
     qw, kw = n_q * dim, n_kv * dim
     q, k = qkv[:, :qw].float(), qkv[:, qw:qw + kw].float()
-    v = qkv[:, qw + kw:qw + kw + n_kv * vdim].float().reshape(T, n_kv, vdim)
+    v_off = qw if v_is_k else qw + kw
+    v = qkv[:, v_off:v_off + n_kv * vdim].float().reshape(T, n_kv, vdim)
     if q_norm is not None:
         q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_norm.float()
     if k_norm is not None:
         k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_norm.float()
     q, k = q.reshape(T, n_q, dim), k.reshape(T, n_kv, dim)
+    if q_temp is not None:
+        q = q * query_temperature(positions, *q_temp)[:, None, None]
     pos = positions.float()[:, None, None]
     r = 2 * inv_freq.numel()
     if r:
@@ -778,20 +794,25 @@ def embed_scale_dyt(tokens, table, scale: float, norm, out_dtype):
 
 
 def residual_post_norm(x, y, post, pre, out_dtype):
-    """``x += post(y)`` in fp32, in place, with ``post`` = ("dyt", alpha, w, b) or ("rms", w, eps)
-    (``y / sqrt(mean(y^2) + eps) * w``); then returns what the next reader of x takes: ``pre`` =
-    ("dyt", alpha, w, b) -> `dyt` of the new x, ("copy",) -> x rounded to ``out_dtype``, None -> None."""
+    """``x += post(y)`` in fp32, in place, with ``post`` = ("dyt", alpha, w, b), ("rms", w, eps)
+    (``y / sqrt(mean(y^2) + eps) * w``) or ("ln", w, b, eps) (`layer_norm32` of y); then returns what the
+    next reader of x takes: ``pre`` = ("dyt", alpha, w, b) -> `dyt` of the new x, ("ln", w, b, eps) (with a
+    layer norm as ``post``) -> its layer norm, ("copy",) -> x rounded to ``out_dtype``, None -> None."""
     yf = y.float()
     if post[0] == "dyt":
         x.add_(torch.tanh(float(post[1]) * yf) * post[2].float() + post[3].float())
     elif post[0] == "rms":
         x.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + float(post[2])) * post[1].float())
+    elif post[0] == "ln":
+        x.add_(layer_norm32(yf, post[1], float(post[3]), torch.float32, post[2]))
     else:
         raise ValueError(f"unknown post norm {post[0]!r}")
     if pre is None:
         return None
     if pre[0] == "copy":
         return x.to(out_dtype)
+    if pre[0] == "ln":
+        return layer_norm32(x, pre[1], float(pre[3]), out_dtype, pre[2])
     return dyt(x, pre[1:], out_dtype)
 
 
@@ -907,11 +928,12 @@ def gelu_gather_mul(z, tokens, table, off: int):
     return (act_fn(z.float(), "gelu_tanh") * e).to(z.dtype)
 
 
-def gated_act(both):
-    """``silu(both[:, :n]) * both[:, n:]`` for a stacked [gate | up] projection [rows, 2 n]; the
-    activation is rounded like a projection's output before the product."""
+def gated_act(both, kind: str = "silu"):
+    """``act(both[:, :n]) * both[:, n:]`` for a stacked [gate | up] projection [rows, 2 n], act of
+    `act_fn` ("silu" | "gelu_tanh"); the activation is rounded like a projection's output before the
+    product."""
     n = both.shape[1] // 2
-    return (act_fn(both[:, :n], "silu").float() * both[:, n:].float()).to(both.dtype)
+    return (act_fn(both[:, :n], kind).float() * both[:, n:].float()).to(both.dtype)
 
 
 # ------------------------------------------------------------------ hyper-connection streams, layer norms, unit-norm rotary
@@ -921,11 +943,12 @@ def gated_act(both):
 # layer norm and its output y is written back as ``X'[t] = sum_s mix[s, t] X[s] + out[t] y``, all
 # streams from the old ones.  S = 1 with read = mix = out = 1 is the plain residual sum.
 
-def layer_norm32(u, w, eps: float, out_dtype):
-    """fp32 ``(u - mean) / sqrt(var + eps) * w`` (biased variance, no bias), rounded once."""
+def layer_norm32(u, w, eps: float, out_dtype, b=None):
+    """fp32 ``(u - mean) / sqrt(var + eps) * w (+ b)`` (biased variance), rounded once."""
     uf = u.float()
     d = uf - uf.mean(-1, keepdim=True)
-    return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
+    y = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+    return (y if b is None else y + b.float()).to(out_dtype)
 
 
 def hyper_embed_norm(tokens, table, streams: int, read_w, norm_w, eps: float, out_dtype):
@@ -1037,3 +1060,17 @@ def moe_route_scored(h, router_w, corr, top: int, groups: int, keep: int, scale:
 def softcap(logits, cap: float):
     """``cap tanh(logits / cap)`` on fp32 logits, in place."""
     return logits.copy_(cap * torch.tanh(logits / cap))
+
+
+# ------------------------------------------------------------------ learned positions (models/sadodra.py)
+
+def embed_position(tokens, positions, table, pos_table, out_dtype):
+    """(fp32 stream ``E[token] + P[position]``, the same rounded to ``out_dtype``)."""
+    x = table.index_select(0, tokens.long()).float() + pos_table.index_select(0, positions.long()).float()
+    return x, x.to(out_dtype)
+
+
+def alibi_slopes(heads: int, device=None) -> torch.Tensor:
+    """fp32 [heads]: ``2^(-8 (h + 1) / heads)``, the distance slopes of biased attention heads."""
+    h = torch.arange(heads, dtype=torch.float64)
+    return torch.pow(2.0, -8.0 * (h + 1.0) / heads).float().to(device)

@@ -9,7 +9,7 @@ synchronise with the host.  Semantics: the functions of the same names in ``refe
 
 import torch
 
-from .seqmix import _act, _check, _p, _req, _stream
+from .seqmix import ACT_CODES, _act, _check, _p, _req, _stream
 from .seqstate import _f32, _i32
 
 
@@ -18,6 +18,9 @@ def _dyt(norm, W):
     _f32(w, W, "dynamic-tanh weight")
     _f32(b, W, "dynamic-tanh bias")
     return float(alpha), _p(w), _p(b)
+
+
+MAX_LN_WIDTH = 16384
 
 
 def seqlatent_ops(lib):
@@ -31,6 +34,25 @@ def seqlatent_ops(lib):
                                        _act(table), _stream()), "embed_scale_dyt")
         return x, h
 
+    def _residual_layer_norm(x, y, post, pre, out_dtype):
+        T, W = x.shape
+        _req(W <= MAX_LN_WIDTH, f"layer-normed residual: width <= {MAX_LN_WIDTH}")
+        _f32(post[1], W, "layer-norm weight")
+        _f32(post[2], W, "layer-norm bias")
+        out, pre_kind, qw, qb, pre_eps = None, 0, None, None, 0.0
+        if pre is not None:
+            out = torch.empty(T, W, dtype=out_dtype, device=x.device)
+            _req(pre[0] in ("copy", "ln"), "behind a layer norm: a rounded copy or a layer norm of the stream")
+            pre_kind = 1
+            if pre[0] == "ln":
+                _f32(pre[1], W, "layer-norm weight")
+                _f32(pre[2], W, "layer-norm bias")
+                pre_kind, qw, qb, pre_eps = 2, _p(pre[1]), _p(pre[2]), float(pre[3])
+        _check(lib.bcg_residual_layer_norm(_p(x), _p(y), int(y.dtype == torch.float32), _p(post[1]), _p(post[2]), float(post[3]),
+                                           pre_kind, qw, qb, pre_eps, _p(out), T, W, int(out_dtype == torch.float32), _stream()),
+               "residual_layer_norm")
+        return out
+
     def residual_post_norm(x, y, post, pre, out_dtype):
         _req(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "residual fp32 [T, W]")
         T, W = x.shape
@@ -41,6 +63,8 @@ def seqlatent_ops(lib):
         elif post[0] == "rms":
             _f32(post[1], W, "norm weight")
             kind, (pa, pw, pb), eps = 1, (0.0, _p(post[1]), None), float(post[2])
+        elif post[0] == "ln":
+            return _residual_layer_norm(x, y, post, pre, out_dtype)
         else:
             raise ValueError(f"unknown post norm {post[0]!r}")
         out, pre_kind, (qa, qw, qb) = None, 0, (0.0, None, None)
@@ -119,10 +143,12 @@ def seqlatent_ops(lib):
                                 group, _act(x), _stream()), "gate_mul")
         return out
 
-    def gated_act(both):
-        _req(both.dim() == 2 and both.is_contiguous() and both.shape[1] % 2 == 0, "gated_act: [rows, 2 n] contiguous")
+    def gated_act(both, kind="silu"):
+        _req(both.dim() == 2 and both.is_contiguous() and both.shape[1] % 2 == 0 and kind in ("silu", "gelu_tanh"),
+             "gated_act: [rows, 2 n] contiguous, silu or gelu_tanh")
         out = torch.empty(both.shape[0], both.shape[1] // 2, dtype=both.dtype, device=both.device)
-        _check(lib.bcg_gated_act(_p(both), _p(out), both.shape[0], both.shape[1] // 2, _act(both), _stream()), "gated_act")
+        _check(lib.bcg_gated_act(_p(both), _p(out), both.shape[0], both.shape[1] // 2, ACT_CODES[kind], _act(both),
+                                 _stream()), "gated_act")
         return out
 
     def ssm_prepare(c, off_b, y, off_dt, dt_bias, a_log, heads, groups, state):

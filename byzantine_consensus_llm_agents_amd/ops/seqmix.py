@@ -37,6 +37,9 @@ def _act(t):
     return int(t.dtype == torch.float32)
 
 
+ACT_CODES = {"gelu_tanh": 0, "relu2": 1, "silu": 2}
+
+
 def seqmix_ops(lib, linear):
     split_keys = lib.bcg_multimap_split_keys()
     tile_rows = lib.bcg_moe_tile_rows()
@@ -51,6 +54,19 @@ def seqmix_ops(lib, linear):
         _check(lib.bcg_embed_scale_rmsnorm(_p(tokens), _p(table), scale, _p(w), eps, w_offset, _p(resid), _p(out), T, W,
                                            table.shape[0], _act(table), _stream()), "embed_scale_rmsnorm")
         return out, resid
+
+    def embed_position(tokens, positions, table, pos_table, out_dtype):
+        _req(tokens.dtype == torch.int32 and tokens.is_contiguous() and tokens.dim() == 1, "tokens int32 [T]")
+        T, W = tokens.numel(), table.shape[1]
+        _req(positions.dtype == torch.int32 and positions.is_contiguous() and positions.numel() == T, "positions int32 [T]")
+        for t in (table, pos_table):
+            _req(t.dim() == 2 and t.is_contiguous() and t.dtype == out_dtype and t.shape[1] == W and t.shape[0] >= 1,
+                 "embedding / position table [rows, W] in the activation dtype")
+        x = torch.empty(T, W, dtype=torch.float32, device=table.device)
+        out = torch.empty(T, W, dtype=out_dtype, device=table.device)
+        _check(lib.bcg_embed_position(_p(tokens), _p(positions), _p(table), _p(pos_table), _p(x), _p(out), T, W, table.shape[0],
+                                      pos_table.shape[0], _act(table), _stream()), "embed_position")
+        return x, out
 
     def residual_add_rmsnorm32(residual, parts, w, eps, w_offset, out_dtype, gate=None, gated=None):
         _req(residual.dtype == torch.float32 and residual.dim() == 2 and residual.is_contiguous(), "residual fp32 [T, W]")
@@ -84,7 +100,7 @@ def seqmix_ops(lib, linear):
         _req(x.dim() == 2 and x.stride(1) == 1, "act_fn: [rows, n] with unit column stride")
         rows, n = x.shape
         out = torch.empty(rows, n, dtype=x.dtype, device=x.device)
-        code = {"gelu_tanh": 0, "relu2": 1, "silu": 2}[kind]
+        code = ACT_CODES[kind]
         _check(lib.bcg_act_fn(_p(x), _p(out), rows, n, x.stride(0), code, _act(x), _stream()), "act_fn")
         return out
 
@@ -138,18 +154,20 @@ def seqmix_ops(lib, linear):
         return 64  # four waves x 16 rows
 
     def multimap_attention(q, k_cache, v_cache, meta, scale, maps, lam, head_eps, out_scale, vdim, window=0, sink=None,
-                           chunk=0):
+                           chunk=0, softcap=0.0, slopes=None):
         """Prefill tiles (``meta.tiles``) on the MFMA kernel, one-token rows (``meta.single``, or
         every row of a decode step) on the split-KV kernel.  ``window`` / ``chunk`` / ``sink``
         (one-map heads): sliding window in keys, or a chunk mask (a query sees the keys of its own
-        ``chunk``-aligned block of positions only); fp32 [H] sink logits of the softmax denominator."""
+        ``chunk``-aligned block of positions only); fp32 [H] sink logits of the softmax denominator.
+        ``softcap`` / ``slopes`` (one-map heads): scaled scores capped by tanh, then fp32 [H] slopes
+        times the distance to the key taken off."""
         T, H, qd = q.shape
         _req(q.is_contiguous() and qd % maps == 0, "q [T, H, maps dim] contiguous")
         dim = qd // maps
         G = k_cache.shape[1]
         NB, BS = _cache_ok(k_cache, v_cache, G, qd, vdim, q.dtype)
-        _req(H % G == 0 and maps in (1, 2) and dim <= (512 if maps == 1 else 128) and vdim <= 256,
-             "multimap attention: maps <= 2, dim <= 128 (one map: 512), vdim <= 256")
+        _req(H % G == 0 and maps in (1, 2) and dim <= (512 if maps == 1 else 128)
+             and vdim <= (512 if maps == 1 else 256), "multimap attention: maps <= 2, dim <= 128 and vdim <= 256 (one map: 512)")
         bt = meta.block_tables
         lens = meta.seq_lens if meta.attn_seq_lens is None else meta.attn_seq_lens
         _req(bt.dtype == torch.int32 and bt.dim() == 2 and bt.is_contiguous() and lens.dtype == torch.int32
@@ -163,7 +181,12 @@ def seqmix_ops(lib, linear):
              and (maps == 1 or (window == 0 and chunk == 0 and sink is None)), "window / chunk / sink: one-map heads, one mask")
         if sink is not None:
             _req(sink.dtype == torch.float32 and sink.numel() == H and sink.is_contiguous(), "sink fp32 [H]")
-        common = (H, G, maps, dim, vdim, BS, NB, scale, lam, head_eps, out_scale, tile_rows, f32, window, chunk, _p(sink), _stream())
+        softcap = float(softcap or 0.0)
+        _req(softcap >= 0 and (maps == 1 or (softcap == 0 and slopes is None)), "softcap / slopes: one-map heads")
+        if slopes is not None:
+            _req(slopes.dtype == torch.float32 and slopes.numel() == H and slopes.is_contiguous(), "slopes fp32 [H]")
+        common = (H, G, maps, dim, vdim, BS, NB, scale, lam, head_eps, out_scale, tile_rows, f32, window, chunk, _p(sink), softcap,
+                  _p(slopes), _stream())
 
         def decode(work, n_items):
             n_splits = max(1, (bt.shape[1] * BS + split_keys - 1) // split_keys)
@@ -257,7 +280,7 @@ def seqmix_ops(lib, linear):
             _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(both), n_up, _p(sorted_), _p(tile_e), n_tiles, n_up, W, top, 1, 0, 0,
                                     f32, _stream()), "moe gate / up")
             hidden = torch.empty(cap, ff, dtype=h.dtype, device=dev)
-            _check(lib.bcg_gated_act(_p(both), _p(hidden), cap, ff, f32, _stream()), "gated_act")
+            _check(lib.bcg_gated_act(_p(both), _p(hidden), cap, ff, ACT_CODES["silu"], f32, _stream()), "gated_act")
         else:
             hidden = torch.empty(cap, ff, dtype=h.dtype, device=dev)
             _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(hidden), ff, _p(sorted_), _p(tile_e), n_tiles, ff, W, top, 1, 0, 1,
@@ -269,7 +292,7 @@ def seqmix_ops(lib, linear):
         _check(lib.bcg_moe_combine(_p(y), _p(weights), _p(out), T, W, top, f32, _stream()), "moe_combine")
         return out
 
-    return dict(embed_scale_rmsnorm=embed_scale_rmsnorm, residual_add_rmsnorm32=residual_add_rmsnorm32,
+    return dict(embed_scale_rmsnorm=embed_scale_rmsnorm, embed_position=embed_position, residual_add_rmsnorm32=residual_add_rmsnorm32,
                 rmsnorm32=rmsnorm32, act_fn=act_fn, rope_multi_kv_write=rope_multi_kv_write,
                 kv_from_logical=kv_from_logical, kv_to_logical=kv_to_logical,
                 multimap_attention=multimap_attention, multimap_tile_rows=multimap_tile_rows, moe_route=moe_route, moe_experts=moe_experts,

@@ -101,10 +101,14 @@ def seqstate_ops(lib):
         return out
 
     def rope_pairs_kv_write(qkv, positions, slots, n_q, n_kv, dim, vdim, q_norm, k_norm, eps, inv_freq, v_inv_freq,
-                            k_cache, v_cache):
+                            k_cache, v_cache, v_is_k=False, q_temp=None):
         T = qkv.shape[0]
         qw, kw, vw = n_q * dim, n_kv * dim, n_kv * vdim
-        _req(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= qw + kw + vw, "row [q | k | v | ...]")
+        _req(not v_is_k or vdim == dim, "values that are the keys: vdim = dim")
+        v_off = qw if v_is_k else qw + kw
+        _req(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] >= max(qw + kw, v_off + vw), "row [q | k | v | ...]")
+        coef, every = (0.0, 0) if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
+        _req(q_temp is None or every >= 1, "query temperature: every >= 1")
         _i32(positions, T, "positions")
         _i32(slots, T, "slots")
         half = inv_freq.numel()
@@ -125,7 +129,7 @@ def seqstate_ops(lib):
         q = torch.empty(T, n_q, dim, dtype=qkv.dtype, device=qkv.device)
         _check(lib.bcg_rope_pairs_kv_write(_p(qkv), qkv.stride(0), _p(positions), _p(slots), _p(q_norm), _p(k_norm), eps,
                                            _p(inv_freq), half, _p(v_inv_freq), _p(q), _p(k_cache), _p(v_cache), T, n_q, n_kv, dim,
-                                           vdim, BS, NB, _act(qkv), _stream()), "rope_pairs_kv_write")
+                                           vdim, v_off, coef, every, BS, NB, _act(qkv), _stream()), "rope_pairs_kv_write")
         return q
 
     def rotate_pairs(x, positions, inv_freq, sign, heads):

@@ -30,6 +30,9 @@
 // floor(j / chunk), chunks counted from position 0), and a per-head sink, a learned logit that takes part in the softmax denominator
 // only (no key, no value, not scaled).  The key loop starts at the window's (chunk's) first 16-key
 // tile; decode splits are counted from the window's (chunk's) first split.
+//
+// Optional score shape (SC instances, one-map heads): the scaled score s becomes cap tanh(s / cap)
+// (cap > 0), then slope_h (i - j) is taken off (slopes non-null).  Both act on fp32 scores.
 #include <algorithm>
 
 #include "seqmix_common.h"
@@ -56,6 +59,8 @@ struct AttnArgs {
   int window;               // > 0: keys below position - window + 1 are hidden
   int chunk;                // > 0: keys below position - position % chunk are hidden (chunks count from position 0)
   const float* sink;        // [H] or null
+  float softcap;            // > 0: scaled scores are capped, cap tanh(s / cap)   (SC instances)
+  const float* slopes;      // [H] or null: slope_h (i - j) is taken off the score (SC instances)
   int swz;                  // fragment-major slabs (see the top of the file)
 };
 
@@ -74,14 +79,16 @@ __device__ __forceinline__ int first_key(const AttnArgs& a, int pos) {
 //   PF         this iteration's V^T fragments are loaded before its QK^T products and the next
 //              iteration's K fragments right after them (loads fly under the MFMAs and the softmax)
 //   FULL       whole, aligned fragments only (no branch around any load)
+//   SC         scores are capped / biased: pos = the position of the lane's column, slope = its head's
+//              slope times log2 e
 // Everything that does not depend on the lane stays scalar: the page lookup and the slab base go
 // to SGPRs, a lane adds a 32-bit offset that is fixed for the whole loop.  Scores are kept in the
 // log2 domain (scale * log2 e folded into one multiply, v_exp_f32 directly).
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int EXACT, int NM>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int EXACT, int NM, bool SC>
 __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const typename Elem<T>::frag (&qf)[NM][KC],
                                              int limit, int limit_min, int lo, int lo_max, int k_begin, int k_last,
                                              const int* __restrict__ table, f32x4 (&acc)[NM][VT], float (&mx)[NM],
-                                             float (&den)[NM]) {
+                                             float (&den)[NM], int pos = 0, float slope = 0.f) {
   typedef typename Elem<T>::frag F;
   // EXACT (1 or 2 = the number of maps): dim = 16 KC, vdim = 16 VT, 16-token pages, fragment-major slabs -- every guard
   // below is a compile-time constant, fragment offsets are immediates, the loop body is straight-line
@@ -98,6 +105,17 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
   const int kc = EXACT ? KC : (a.dim + 15) >> 4, vt = EXACT ? VT : (a.vdim + 15) >> 4;
   const bool vec_k = a.vec_k && (a.dim & 3) == 0;
   const float sc = a.scale * 1.4426950408889634f;
+  // capped scores: cap tanh(s / cap) = cap - 2 cap / (exp(2 s / cap) + 1), in the log2 domain
+  const float cap = SC ? a_.softcap : 0.f;
+  const float cap2 = cap * LOG2E, arg2 = cap > 0.f ? 2.0f * LOG2E * a.scale / cap : 0.f;
+  auto shape_score = [&](float dot, int key, bool capped) {
+    float v = dot * sc;
+    if (capped) {
+      if constexpr (sizeof(T) == 2) v = cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot * arg2) + 1.0f);
+      else v = cap2 * tanhf(dot * a.scale / cap);
+    }
+    return v - slope * static_cast<float>(pos - key);
+  };
   // offsets inside a (page, KV head) slab = one lane offset (fixed for the whole loop) + a
   // wave-uniform offset per fragment; the slab base and the tile's key offset are uniform too
   const uint32_t k_lane = a.swz ? (grp * a.BS + col) * 4 : col * KD + 4 * grp;
@@ -179,6 +197,10 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
     if (PF && key0 + 16 * KT <= k_last) load_k(k_cur, kf);
     // ---- online softmax per query column; lane holds keys key0 + 16 u + 4 grp + i ----
     const bool masked = key0 + 16 * KT - 1 > limit_min || key0 < lo_max;   // (wave-uniform) some key of the iteration is hidden
+    // (opaque per iteration: one loop body, not one per combination of uniform conditions)
+    float cap_now = cap;
+    if constexpr (SC) asm volatile("" : "+v"(cap_now));
+    const bool capped = cap_now > 0.f;
     F pf[KT][NM];
 #pragma unroll
     for (int m = 0; m < NM; ++m) {
@@ -192,7 +214,8 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
       for (int u = 0; u < KT; ++u)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          v[u][i] = s[u][m][i] * sc;
+          if constexpr (SC) v[u][i] = shape_score(s[u][m][i], key0 + 16 * u + 4 * grp + i, capped);
+          else v[u][i] = s[u][m][i] * sc;
           if (masked && (key0 + 16 * u + 4 * grp + i > limit || key0 + 16 * u + 4 * grp + i < lo)) v[u][i] = -INFINITY;
           bm = fmaxf(bm, v[u][i]);
         }
@@ -237,7 +260,7 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
   }
 }
 
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, bool SC = false>
 __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
   typedef typename Elem<T>::frag F;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -280,8 +303,9 @@ __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
   }
   const int lo = first_key(a, pos), lo_max = first_key(a, pos_max);   // (both masks: the first key grows with the position)
   const int k_begin = first_key(a, pos_min) & ~15;
-  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM>(a, g, qf, pos, pos_min, lo, lo_max, k_begin, pos_max,
-                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den);
+  const float slope = SC && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
+  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, SC>(a, g, qf, pos, pos_min, lo, lo_max, k_begin, pos_max,
+                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, pos, slope);
   // ---- combine the maps, unit norm over the head's value features, store ----
   const float i0 = 1.0f / den[0];
   float i1 = 0.f;
@@ -323,7 +347,7 @@ __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
 // head g (H / G) + 16 cg + c of the same token, so K and V^T are read once per KV head.  One wave
 // per (item, KV head x column group, SPLIT_KEYS-key split); partials as the merge kernel reads them
 // (running maxima in the log2 domain of `attend_range`).
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, bool SC = false>
 __global__ __launch_bounds__(64, OCC) void decode_mfma_kernel(AttnArgs a) {
   typedef typename Elem<T>::frag F;
   const int lane = threadIdx.x, col = lane & 15, grp = lane >> 4;
@@ -362,8 +386,9 @@ __global__ __launch_bounds__(64, OCC) void decode_mfma_kernel(AttnArgs a) {
     mx[m] = MAX_FLOOR;
     den[m] = 0.f;
   }
-  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM>(a, g, qf, k_end - 1, k_end - 1, lo, lo, k_begin, k_end - 1,
-                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den);
+  const float slope = SC && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
+  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, SC>(a, g, qf, k_end - 1, k_end - 1, lo, lo, k_begin, k_end - 1,
+                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, ctx - 1, slope);
   if (!col_ok) return;
   float* w = a.ws + ((static_cast<size_t>(item) * a.H + h) * a.n_splits + split) * (2 * a.maps + a.maps * a.vdim);
 #pragma unroll
@@ -431,20 +456,61 @@ __global__ __launch_bounds__(64) void decode_merge_kernel(AttnArgs a) {
   }
 }
 
+// Exact one-map instances (bf16): X(KC, VT, keys tiles per iteration, workgroups per CU).
+#define BCG_EXACT1_PLAIN(X) X(8, 8, 2, 2) X(4, 4, 2, 2) X(4, 8, 2, 2) X(2, 2, 2, 2) X(6, 6, 2, 2) X(6, 4, 2, 2) X(12, 8, 2, 2) \
+                            X(12, 12, 2, 1) X(16, 16, 2, 1) X(32, 32, 1, 1)
+#define BCG_EXACT1_SHAPED(X) X(8, 8, 2, 2) X(4, 4, 2, 2) X(2, 2, 2, 2) X(3, 3, 2, 2) X(6, 6, 2, 2) X(12, 12, 2, 1) X(16, 16, 2, 1)
+
+// Heads whose scores are capped or biased (one map).
+template <typename T>
+int launch_prefill_shaped(const AttnArgs& a, int n_tiles, bool full, hipStream_t s) {
+  dim3 grid(n_tiles, a.H);
+  if constexpr (sizeof(T) == 2) if (full && a.swz && a.BS == 16) {
+#define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
+  if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
+    prefill_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, true><<<grid, 256, 0, s>>>(a);      \
+    return BCG_CHECK_LAUNCH();                                                                   \
+  }
+    BCG_EXACT1_SHAPED(BCG_X)
+#undef BCG_X
+  }
+  if (a.dim <= 64 && a.vdim <= 128) prefill_kernel<T, 4, 8, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
+  else if (a.dim <= 256 && a.vdim <= 256) prefill_kernel<T, 16, 16, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
+  else prefill_kernel<T, 32, 32, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
+  return BCG_CHECK_LAUNCH();
+}
+
+template <typename T>
+void launch_decode_shaped(const AttnArgs& a, dim3 grid, bool full, hipStream_t s) {
+  if constexpr (sizeof(T) == 2) if (full && a.swz && a.BS == 16) {
+#define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
+  if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
+    decode_mfma_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, true><<<grid, 64, 0, s>>>(a);   \
+    return;                                                                                      \
+  }
+    BCG_EXACT1_SHAPED(BCG_X)
+#undef BCG_X
+  }
+  if (a.dim <= 64 && a.vdim <= 128) decode_mfma_kernel<T, 4, 8, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
+  else if (a.dim <= 256 && a.vdim <= 256) decode_mfma_kernel<T, 16, 16, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
+  else decode_mfma_kernel<T, 32, 32, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
+}
+
 template <typename T>
 int launch_prefill(const AttnArgs& a, int n_tiles, int tile_rows, hipStream_t s) {
   dim3 grid(n_tiles, a.H);
   const bool small = a.dim <= 64 && a.vdim <= 128;
   const bool full = a.dim % 16 == 0 && a.vdim % 16 == 0 && a.vec_k && a.vec_v;   // whole, aligned fragments only
   if (tile_rows != 64) return -2;
+  if (a.softcap > 0.f || a.slopes != nullptr) return launch_prefill_shaped<T>(a, n_tiles, full, s);
   if constexpr (sizeof(T) == 2) if (full && a.maps == 1 && a.swz && a.BS == 16) {   // one-map heads, exact shapes
-#define BCG_EXACT1(KC_, VT_)                                                                     \
+#define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
-    prefill_kernel<T, KC_, VT_, 2, true, true, 2, 1, 1><<<grid, 256, 0, s>>>(a);                 \
+    prefill_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1><<<grid, 256, 0, s>>>(a);            \
     return BCG_CHECK_LAUNCH();                                                                   \
   }
-    BCG_EXACT1(8, 8) BCG_EXACT1(4, 4) BCG_EXACT1(4, 8) BCG_EXACT1(2, 2) BCG_EXACT1(6, 6) BCG_EXACT1(6, 4) BCG_EXACT1(12, 8)
-#undef BCG_EXACT1
+    BCG_EXACT1_PLAIN(BCG_X)
+#undef BCG_X
   }
   if constexpr (sizeof(T) == 2) if (small) {
     const bool exact = full && a.maps == 2 && a.swz && a.BS == 16;
@@ -462,6 +528,8 @@ int launch_prefill(const AttnArgs& a, int n_tiles, int tile_rows, hipStream_t s)
   if (small) {
     if (full) prefill_kernel<T, 4, 8, 1, false, true, 2><<<grid, 256, 0, s>>>(a);
     else prefill_kernel<T, 4, 8, 1, false, false, 2><<<grid, 256, 0, s>>>(a);
+  } else if (a.vdim > 256) {   // one map of more than 256 value features (a wide latent)
+    prefill_kernel<T, 32, 32, 1, false, false, 1, 0, 1><<<grid, 256, 0, s>>>(a);
   } else if (a.dim <= 128) {   // (the branch-free form of the wide instance runs out of registers)
     prefill_kernel<T, 8, 16, 1, false, false, 1><<<grid, 256, 0, s>>>(a);
   } else if (a.dim <= 256) {   // one map of up to 256 key features (a latent plus a rotated part)
@@ -477,15 +545,16 @@ int launch_decode(const AttnArgs& a, int n_items, hipStream_t s) {
   const int per = a.H / a.G;
   dim3 grid(a.G * ((per + 15) / 16), a.n_splits, n_items);
   const bool full = a.dim % 16 == 0 && a.vdim % 16 == 0 && a.vec_k && a.vec_v;
-  bool done = false;
-  if constexpr (sizeof(T) == 2) if (full && a.maps == 1 && a.swz && a.BS == 16) {   // one-map heads, exact shapes
-#define BCG_EXACT1(KC_, VT_)                                                                     \
+  bool done = a.softcap > 0.f || a.slopes != nullptr;
+  if (done) launch_decode_shaped<T>(a, grid, full, s);
+  if constexpr (sizeof(T) == 2) if (!done && full && a.maps == 1 && a.swz && a.BS == 16) {   // one-map heads, exact shapes
+#define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (!done && a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                        \
     done = true;                                                                                 \
-    decode_mfma_kernel<T, KC_, VT_, 2, true, true, 2, 1, 1><<<grid, 64, 0, s>>>(a);              \
+    decode_mfma_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1><<<grid, 64, 0, s>>>(a);         \
   }
-    BCG_EXACT1(8, 8) BCG_EXACT1(4, 4) BCG_EXACT1(4, 8) BCG_EXACT1(2, 2) BCG_EXACT1(6, 6) BCG_EXACT1(6, 4) BCG_EXACT1(12, 8)
-#undef BCG_EXACT1
+    BCG_EXACT1_PLAIN(BCG_X)
+#undef BCG_X
   }
   if constexpr (sizeof(T) == 2) if (!done && a.dim <= 64 && a.vdim <= 128) {
     done = true;
@@ -507,6 +576,8 @@ int launch_decode(const AttnArgs& a, int n_items, hipStream_t s) {
   } else if (a.dim <= 64 && a.vdim <= 128) {
     if (full) decode_mfma_kernel<T, 4, 8, 1, false, true, 2><<<grid, 64, 0, s>>>(a);
     else decode_mfma_kernel<T, 4, 8, 1, false, false, 2><<<grid, 64, 0, s>>>(a);
+  } else if (a.vdim > 256) {
+    decode_mfma_kernel<T, 32, 32, 1, false, false, 1, 0, 1><<<grid, 64, 0, s>>>(a);
   } else if (a.dim <= 128) {
     decode_mfma_kernel<T, 8, 16, 1, false, false, 1><<<grid, 64, 0, s>>>(a);
   } else if (a.dim <= 256) {
@@ -515,7 +586,8 @@ int launch_decode(const AttnArgs& a, int n_items, hipStream_t s) {
     decode_mfma_kernel<T, 32, 16, 1, false, false, 1, 0, 1><<<grid, 64, 0, s>>>(a);
   }
   if (a.vdim <= 128) decode_merge_kernel<T, 2><<<dim3(a.H, n_items), 64, 0, s>>>(a);
-  else decode_merge_kernel<T, 4><<<dim3(a.H, n_items), 64, 0, s>>>(a);
+  else if (a.vdim <= 256) decode_merge_kernel<T, 4><<<dim3(a.H, n_items), 64, 0, s>>>(a);
+  else decode_merge_kernel<T, 8><<<dim3(a.H, n_items), 64, 0, s>>>(a);
   return BCG_CHECK_LAUNCH();
 }
 
@@ -530,11 +602,11 @@ BCG_API int bcg_multimap_attention(int mode, const void* q, const void* k_cache,
                                    const void* work, int n_work, void* out, void* ws, int n_splits, int H, int G, int maps,
                                    int dim, int vdim, int BS, int num_blocks, float scale, float lam, float head_eps,
                                    float out_scale, int tile_rows, int is_f32, int window, int chunk, const void* sink,
-                                   void* stream) {
+                                   float softcap, const void* slopes, void* stream) {
   if (n_work <= 0) return 0;
-  if ((window > 0 || chunk > 0 || sink != nullptr) && maps != 1) return -2;
+  if ((window > 0 || chunk > 0 || sink != nullptr || softcap != 0.f || slopes != nullptr) && maps != 1) return -2;
   if (window > 0 && chunk > 0) return -2;
-  if (maps < 1 || maps > 2 || dim > (maps == 1 ? 512 : 128) || vdim > 256 || BS % 16 || H % G || n_work > 65535 * 16) return -2;
+  if (maps < 1 || maps > 2 || dim > (maps == 1 ? 512 : 128) || vdim > (maps == 1 ? 512 : 256) || BS % 16 || H % G || n_work > 65535 * 16) return -2;
   AttnArgs a;
   a.q = q; a.k_cache = k_cache; a.v_cache = v_cache;
   a.block_tables = static_cast<const int*>(block_tables); a.q_start = static_cast<const int*>(q_start);
@@ -547,6 +619,7 @@ BCG_API int bcg_multimap_attention(int mode, const void* q, const void* k_cache,
   a.vec_v = 1;  // BS % 16 == 0: every 4-key group of a V^T row is aligned
   a.swz = a.vec_k;
   a.window = window; a.chunk = chunk; a.sink = static_cast<const float*>(sink);
+  a.softcap = softcap; a.slopes = static_cast<const float*>(slopes);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (mode == 0) return is_f32 ? launch_prefill<float>(a, n_work, tile_rows, s) : launch_prefill<bf16_t>(a, n_work, tile_rows, s);
   if (n_splits < 1 || H > 65535 || n_splits > 65535 || n_work > 65535) return -2;

@@ -32,6 +32,7 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float siluf_(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float siluf_arg(float z, float u) { return z / (1.0f + expf(-u)); }   // z sigmoid(u)
 __device__ __forceinline__ float softplusf_(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float gelu_tanhf_(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
@@ -128,6 +129,91 @@ __global__ __launch_bounds__(NT) void residual_post_norm_kernel(float* __restric
     resid[base + i] = x;
     if (pre_kind == 1) out[base + i] = Elem<T>::st(x);
     else if (pre_kind == 2) out[base + i] = Elem<T>::st(dyt(pre, x, i));
+  }
+}
+
+// ---------------------------------------------------------------- x += layer_norm(y); out = x rounded | layer_norm(x)
+// One workgroup per row, which stays in registers: NV chunks of V columns per thread (NV * V * NT >= W;
+// V = 4: 8- / 16-byte accesses).  pre_kind 0: nothing; 1: x rounded to T; 2: the layer norm (qw, qb) of
+// the new x.  Mean first, then the squared deviations.
+template <typename T, typename Y, int V, int NV>
+__global__ __launch_bounds__(NT) void residual_layer_norm_kernel(float* __restrict__ resid, const Y* __restrict__ y,
+                                                                 const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                                 int pre_kind, const float* __restrict__ qw,
+                                                                 const float* __restrict__ qb, float pre_eps, T* __restrict__ out,
+                                                                 int W) {
+  __shared__ float red[NT / 64];
+  const size_t base = static_cast<size_t>(blockIdx.x) * W;
+  float v[NV][V];
+  auto stats = [&](float e, float& mean, float& r) {
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+#pragma unroll
+      for (int j = 0; j < V; ++j) s += v[k][j];   // (columns past the row hold zeros)
+    mean = block_sum(s, red) / W;
+    float sq = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+      if (V * (threadIdx.x + k * NT) < W) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          const float d = v[k][j] - mean;
+          sq += d * d;
+        }
+      }
+    r = 1.0f / sqrtf(block_sum(sq, red) / W + e);
+  };
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = V * (threadIdx.x + k * NT);
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[k][j] = 0.f;
+    if (i < W) {
+      if constexpr (V == 4) {
+        const typename Vec4<Y>::type f = *reinterpret_cast<const typename Vec4<Y>::type*>(y + base + i);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[k][j] = Elem<Y>::ld(f[j]);
+      } else {
+        v[k][0] = Elem<Y>::ld(y[base + i]);
+      }
+    }
+  }
+  float mean, r;
+  stats(eps, mean, r);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = V * (threadIdx.x + k * NT);
+    if (i < W) {
+      if constexpr (V == 4) {
+        f32x4 x = *reinterpret_cast<const f32x4*>(resid + base + i);
+        const f32x4 pw = *reinterpret_cast<const f32x4*>(w + i), pb = *reinterpret_cast<const f32x4*>(b + i);
+        typename Vec4<T>::type o;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          x[j] += (v[k][j] - mean) * r * pw[j] + pb[j];
+          v[k][j] = x[j];
+          o[j] = Elem<T>::st(x[j]);
+        }
+        *reinterpret_cast<f32x4*>(resid + base + i) = x;
+        if (pre_kind == 1) *reinterpret_cast<typename Vec4<T>::type*>(out + base + i) = o;
+      } else {
+        const float x = resid[base + i] + (v[k][0] - mean) * r * w[i] + b[i];
+        v[k][0] = x;
+        resid[base + i] = x;
+        if (pre_kind == 1) out[base + i] = Elem<T>::st(x);
+      }
+    }
+  }
+  if (pre_kind != 2) return;
+  stats(pre_eps, mean, r);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = V * (threadIdx.x + k * NT);
+    if (i < W) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) out[base + i + j] = Elem<T>::st((v[k][j] - mean) * r * qw[i + j] + qb[i + j]);
+    }
   }
 }
 
@@ -250,16 +336,38 @@ __global__ __launch_bounds__(NT) void gate_mul_kernel(const T* __restrict__ x, c
   }
 }
 
-// out[r, c] = silu(in[r, c]) * in[r, n + c]: the hidden activation of a gated expert from its
+// The activations of bcg_act_fn that gate: kind 0 gelu (tanh form), 2 silu.  gelu as z sigmoid(2 u),
+// which is 0.5 z (1 + tanh(u)).
+__device__ __forceinline__ float gate_act(float z, int kind) {
+  return kind == 0 ? siluf_arg(z, 1.5957691216057308f * (z + 0.044715f * z * z * z)) : siluf_(z);
+}
+
+// out[r, c] = act(in[r, c]) * in[r, n + c], four columns per thread (n a multiple of 4, aligned):
+// blockIdx.y walks the rows.
+template <typename T>
+__global__ __launch_bounds__(NT) void gated_act_vec_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind) {
+  typedef typename Vec4<T>::type VT;
+  const int c = 4 * (blockIdx.x * NT + threadIdx.x);
+  if (c >= n) return;
+  for (int64_t r = blockIdx.y; r < rows; r += gridDim.y) {
+    const VT g = *reinterpret_cast<const VT*>(in + r * 2 * n + c), u = *reinterpret_cast<const VT*>(in + r * 2 * n + n + c);
+    VT o;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = Elem<T>::st(Elem<T>::ld(Elem<T>::st(gate_act(Elem<T>::ld(g[j]), kind))) * Elem<T>::ld(u[j]));
+    *reinterpret_cast<VT*>(out + r * n + c) = o;
+  }
+}
+
+// out[r, c] = act(in[r, c]) * in[r, n + c]: the hidden activation of a gated feed-forward from its
 // stacked [gate | up] projection.
 template <typename T>
-__global__ __launch_bounds__(NT) void gated_act_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n) {
+__global__ __launch_bounds__(NT) void gated_act_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind) {
   const int64_t total = rows * n;
   for (int64_t e = static_cast<int64_t>(blockIdx.x) * NT + threadIdx.x; e < total; e += static_cast<int64_t>(gridDim.x) * NT) {
     const int64_t r = e / n;
     const int c = static_cast<int>(e - r * n);
     // rounded as a projection's output before the product, like every other activation
-    const float g = Elem<T>::ld(Elem<T>::st(siluf_(Elem<T>::ld(in[r * 2 * n + c]))));
+    const float g = Elem<T>::ld(Elem<T>::st(gate_act(Elem<T>::ld(in[r * 2 * n + c]), kind)));
     out[e] = Elem<T>::st(g * Elem<T>::ld(in[r * 2 * n + n + c]));
   }
 }
@@ -379,6 +487,39 @@ BCG_API int bcg_residual_post_norm(void* resid, const void* y, int y_f32, int po
   return BCG_CHECK_LAUNCH();
 }
 
+// x += layer_norm(y) (w, b, eps); pre_kind 0 / 1 / 2: nothing / rounded copy / layer norm (qw, qb,
+// pre_eps) of the new x.  y_f32: y is float whatever the activation type.  W <= 16384.
+BCG_API int bcg_residual_layer_norm(void* resid, const void* y, int y_f32, const void* w, const void* b, float eps, int pre_kind,
+                                    const void* qw, const void* qb, float pre_eps, void* out, int T_, int W, int is_f32,
+                                    void* stream) {
+  if (T_ <= 0) return 0;
+  if (W < 1 || W > 16384 || pre_kind < 0 || pre_kind > 2 || w == nullptr || b == nullptr) return -2;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const float *wf = static_cast<const float*>(w), *bf = static_cast<const float*>(b), *qwf = static_cast<const float*>(qw),
+              *qbf = static_cast<const float*>(qb);
+  auto al16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = W % 4 == 0 && al16(resid) && al16(y) && al16(out) && al16(w) && al16(b);
+#define BCG_RLN(TYPE, YTYPE, V, NV)                                                                                          \
+  residual_layer_norm_kernel<TYPE, YTYPE, V, NV><<<T_, NT, 0, s>>>(static_cast<float*>(resid), static_cast<const YTYPE*>(y), wf, \
+                                                                   bf, eps, pre_kind, qwf, qbf, pre_eps, static_cast<TYPE*>(out), W)
+#define BCG_RLN_BY_WIDTH(TYPE, YTYPE)                                                    \
+  do {                                                                                   \
+    if (vec && W <= 4 * NT) BCG_RLN(TYPE, YTYPE, 4, 1);                                  \
+    else if (vec && W <= 8 * NT) BCG_RLN(TYPE, YTYPE, 4, 2);                             \
+    else if (vec && W <= 16 * NT) BCG_RLN(TYPE, YTYPE, 4, 4);                            \
+    else if (vec && W <= 32 * NT) BCG_RLN(TYPE, YTYPE, 4, 8);                            \
+    else if (vec) BCG_RLN(TYPE, YTYPE, 4, 16);                                           \
+    else if (W <= 4 * NT) BCG_RLN(TYPE, YTYPE, 1, 4);                                    \
+    else BCG_RLN(TYPE, YTYPE, 1, 64);                                                    \
+  } while (0)
+  if (is_f32) BCG_RLN_BY_WIDTH(float, float);
+  else if (y_f32) BCG_RLN_BY_WIDTH(bf16_t, float);
+  else BCG_RLN_BY_WIDTH(bf16_t, bf16_t);
+#undef BCG_RLN_BY_WIDTH
+#undef BCG_RLN
+  return BCG_CHECK_LAUNCH();
+}
+
 BCG_API int bcg_rmsnorm_cols(const void* y, int64_t stride, int off, int n, const void* w, float eps, void* out, int T_,
                              int is_f32, void* stream) {
   if (T_ <= 0 || n <= 0) return 0;
@@ -434,11 +575,18 @@ BCG_API int bcg_gate_mul(const void* x, const void* gate, int64_t gate_stride, v
   return BCG_CHECK_LAUNCH();
 }
 
-BCG_API int bcg_gated_act(const void* in, void* out, int64_t rows, int n, int is_f32, void* stream) {
+BCG_API int bcg_gated_act(const void* in, void* out, int64_t rows, int n, int kind, int is_f32, void* stream) {
   if (rows <= 0 || n <= 0) return 0;
+  if (kind != 0 && kind != 2) return -2;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  BCG_BY_TYPE((gated_act_kernel<float><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n)),
-              (gated_act_kernel<bf16_t><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n)));
+  if (n % 4 == 0 && ((reinterpret_cast<uintptr_t>(in) | reinterpret_cast<uintptr_t>(out)) & 15) == 0) {
+    const dim3 grid((n / 4 + NT - 1) / NT, static_cast<unsigned>(std::min<int64_t>(rows, 65535)));
+    BCG_BY_TYPE((gated_act_vec_kernel<float><<<grid, NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind)),
+                (gated_act_vec_kernel<bf16_t><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind)));
+    return BCG_CHECK_LAUNCH();
+  }
+  BCG_BY_TYPE((gated_act_kernel<float><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind)),
+              (gated_act_kernel<bf16_t><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind)));
   return BCG_CHECK_LAUNCH();
 }
 

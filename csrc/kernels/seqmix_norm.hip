@@ -1,4 +1,4 @@
-// fp32 residual stream: scaled embedding + norm, sublayer sum + residual add + next norm,
+// fp32 residual stream: scaled embedding + norm, embedding + learned position, sublayer sum + residual add + next norm,
 // activations, partial rotary with multi-map heads + paged K / V^T write.
 //
 // The residual stream x is fp32 whatever the activation type T (bf16 bits or float); norms
@@ -41,6 +41,46 @@ __global__ __launch_bounds__(NT) void embed_scale_norm_kernel(const int* __restr
   const float r = 1.0f / sqrtf(block_sum(ss, red) / W + eps);
   T* o = out + static_cast<size_t>(t) * W;
   for (int i = threadIdx.x; i < W; i += NT) o[i] = Elem<T>::st(x[i] * r * (w_offset + w[i]));
+}
+
+// x = table[token] + pos_table[position] (both of type T, summed in fp32), out = x rounded to T.
+// VEC: four columns per thread (W a multiple of 4, aligned tables).
+template <typename T, bool VEC>
+__global__ __launch_bounds__(NT) void embed_position_kernel(const int* __restrict__ tokens, const int* __restrict__ positions,
+                                                            const T* __restrict__ table, const T* __restrict__ pos_table,
+                                                            float* __restrict__ resid, T* __restrict__ out, int W, int vocab,
+                                                            int max_pos) {
+  typedef typename Elem<T>::frag F;
+  const int t = blockIdx.x;
+  const int tok = min(max(tokens[t], 0), vocab - 1), pos = min(max(positions[t], 0), max_pos - 1);
+  const T *a = table + static_cast<size_t>(tok) * W, *b = pos_table + static_cast<size_t>(pos) * W;
+  float* x = resid + static_cast<size_t>(t) * W;
+  T* o = out + static_cast<size_t>(t) * W;
+  if constexpr (VEC) {
+    for (int i = 4 * threadIdx.x; i < W; i += 4 * NT) {
+      const F fa = *reinterpret_cast<const F*>(a + i), fb = *reinterpret_cast<const F*>(b + i);
+      f32x4 v;
+      F r;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if constexpr (sizeof(T) == 2) {
+          v[j] = bf2f(static_cast<bf16_t>(fa[j])) + bf2f(static_cast<bf16_t>(fb[j]));
+          r[j] = static_cast<short>(f2bf(v[j]));
+        } else {
+          v[j] = fa[j] + fb[j];
+          r[j] = v[j];
+        }
+      }
+      *reinterpret_cast<f32x4*>(x + i) = v;
+      *reinterpret_cast<F*>(o + i) = r;
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += NT) {
+      const float v = Elem<T>::ld(a[i]) + Elem<T>::ld(b[i]);
+      x[i] = v;
+      o[i] = Elem<T>::st(v);
+    }
+  }
 }
 
 // x += (p0 + p1 + pf + sigmoid(gate) * pg); out = norm(x) (w == nullptr: no norm).
@@ -161,6 +201,26 @@ BCG_API int bcg_embed_scale_rmsnorm(const void* tokens, const void* table, float
     embed_scale_norm_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const int*>(tokens), static_cast<const bf16_t*>(table), scale,
                                                      static_cast<const float*>(w), eps, w_offset,
                                                      static_cast<float*>(resid), static_cast<bf16_t*>(out), W, vocab);
+  return BCG_CHECK_LAUNCH();
+}
+
+BCG_API int bcg_embed_position(const void* tokens, const void* positions, const void* table, const void* pos_table, void* resid,
+                               void* out, int T_, int W, int vocab, int max_pos, int is_f32, void* stream) {
+  if (T_ <= 0) return 0;
+  if (vocab < 1 || max_pos < 1) return -2;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const int *tk = static_cast<const int*>(tokens), *ps = static_cast<const int*>(positions);
+  auto al16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = W % 4 == 0 && al16(table) && al16(pos_table) && al16(resid) && al16(out);
+#define BCG_EMBED(TYPE, VEC)                                                                                              \
+  embed_position_kernel<TYPE, VEC><<<T_, NT, 0, s>>>(tk, ps, static_cast<const TYPE*>(table), static_cast<const TYPE*>(pos_table), \
+                                                     static_cast<float*>(resid), static_cast<TYPE*>(out), W, vocab, max_pos)
+  if (is_f32) {
+    if (vec) BCG_EMBED(float, true); else BCG_EMBED(float, false);
+  } else {
+    if (vec) BCG_EMBED(bf16_t, true); else BCG_EMBED(bf16_t, false);
+  }
+#undef BCG_EMBED
   return BCG_CHECK_LAUNCH();
 }
 

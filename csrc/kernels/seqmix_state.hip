@@ -36,6 +36,11 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
 
+// Factor of the query at position p: 1 + coef ln(floor((p + 1) / every) + 1) (every = 0: 1).
+__device__ __forceinline__ float query_temperature(int p, float coef, int every) {
+  return every > 0 ? 1.0f + coef * logf(static_cast<float>((p + 1) / every + 1)) : 1.0f;
+}
+
 // ---------------------------------------------------------------- embedding + hashed bigram + scalar norms
 template <typename T>
 __global__ __launch_bounds__(NT) void embed_bigram_kernel(const int* __restrict__ tokens, const int* __restrict__ positions,
@@ -268,7 +273,8 @@ __global__ __launch_bounds__(NT) void short_conv_state_kernel(const T* __restric
 // RMS-normed over their whole width (weights q_norm / k_norm; null = as they are); features
 // (2i, 2i + 1), i < half, of every q / k head turn by position * inv_freq[i]; every pair of every v
 // head by position * v_inv_freq[i] (null = as they are).  K / V^T go to the paged cache in the
-// slab layout of seqmix_attention.hip (one map).
+// slab layout of seqmix_attention.hip (one map).  The values start at column v_off (at the k part
+// itself when the values are the keys before their norm); q is also multiplied by its temperature.
 template <typename T>
 __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__ qkv, int64_t row_stride,
                                                            const int* __restrict__ positions, const int* __restrict__ slots,
@@ -276,7 +282,8 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
                                                            float eps, const float* __restrict__ inv_freq, int half,
                                                            const float* __restrict__ v_inv_freq, T* __restrict__ q_out,
                                                            T* __restrict__ k_cache, T* __restrict__ v_cache, int n_q, int n_kv,
-                                                           int dim, int vdim, int BS, int num_blocks) {
+                                                           int dim, int vdim, int v_off, float temp_coef, int temp_every,
+                                                           int BS, int num_blocks) {
   __shared__ float red[NT / 64];
   const int t = blockIdx.x;
   const T* row = qkv + static_cast<size_t>(t) * row_stride;
@@ -302,6 +309,7 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
     }
     rk = 1.0f / sqrtf(block_sum(s, red) / kw + eps);
   }
+  rq *= query_temperature(positions[t], temp_coef, temp_every);
   const bool swz = (dim & 3) == 0;
   for (int idx = threadIdx.x; idx < qw + kw; idx += NT) {
     const bool is_q = idx < qw;
@@ -326,7 +334,7 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
     }
   }
   if (kv_ok) {
-    const T* vrow = row + qw + kw;
+    const T* vrow = row + v_off;
     for (int idx = threadIdx.x; idx < vw; idx += NT) {
       const int g = idx / vdim, e = idx - g * vdim;
       float val = Elem<T>::ld(vrow[idx]);
@@ -339,6 +347,114 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
       T* slab = v_cache + (static_cast<size_t>(blk) * n_kv + g) * vdim * BS;
       if (swz) slab[(static_cast<size_t>(off >> 2) * vdim + e) * 4 + (off & 3)] = Elem<T>::st(val);
       else slab[static_cast<size_t>(e) * BS + off] = Elem<T>::st(val);
+    }
+  }
+}
+
+// The same without any rotation (half = 0, values as they are), four features per access: dim, vdim,
+// the row stride and the row's start are multiples of four elements.  TPB tokens per workgroup:
+// 4 (a wave per token; four tokens on consecutive slots of one 4-key group write their values as
+// whole groups) for large steps, 1 for small ones.
+template <typename T, int TPB>
+__global__ __launch_bounds__(NT) void norm_kv_kernel(const T* __restrict__ qkv, int64_t row_stride, const int* __restrict__ positions,
+                                                     const int* __restrict__ slots, const float* __restrict__ q_norm,
+                                                     const float* __restrict__ k_norm, float eps, T* __restrict__ q_out,
+                                                     T* __restrict__ k_cache, T* __restrict__ v_cache, int n_q, int n_kv, int dim,
+                                                     int vdim, int v_off, float temp_coef, int temp_every, int BS, int num_blocks,
+                                                     int n_tokens) {
+  typedef typename Elem<T>::frag F;
+  constexpr int TPT = NT / TPB;   // threads per token
+  __shared__ float red[2][NT / 64];
+  const int sub = threadIdx.x / TPT, tid = threadIdx.x - sub * TPT;
+  const int t = blockIdx.x * TPB + sub;
+  const bool live = t < n_tokens;
+  const int qw = n_q * dim, kw = n_kv * dim, vw = n_kv * vdim;
+  const T* row = qkv + static_cast<size_t>(live ? t : n_tokens - 1) * row_stride;
+  auto get = [](const F& f, int j) {
+    if constexpr (sizeof(T) == 2) return bf2f(static_cast<bf16_t>(f[j])); else return f[j];
+  };
+  float sq = 0.f, sk = 0.f;
+  for (int i = 4 * tid; i < qw + kw; i += 4 * TPT) {
+    const F f = *reinterpret_cast<const F*>(row + i);
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) s += get(f, j) * get(f, j);
+    if (i < qw) sq += s; else sk += s;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if constexpr (TPB == 1) {
+    if ((threadIdx.x & 63) == 0) {
+      red[0][threadIdx.x >> 6] = sq;
+      red[1][threadIdx.x >> 6] = sk;
+    }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < NT / 64; ++i) {
+      sq += red[0][i];
+      sk += red[1][i];
+    }
+  }
+  const float rk = k_norm != nullptr ? 1.0f / sqrtf(sk / kw + eps) : 1.0f;
+  const float rq = (q_norm != nullptr ? 1.0f / sqrtf(sq / qw + eps) : 1.0f) *
+                   query_temperature(live ? positions[t] : 0, temp_coef, temp_every);
+  const int slot = live ? slots[t] : -1;
+  const int blk = slot / BS, off = slot - blk * BS;
+  const bool kv_ok = slot >= 0 && blk < num_blocks;
+  if (live) {
+    for (int i = 4 * tid; i < qw + kw; i += 4 * TPT) {
+      const F f = *reinterpret_cast<const F*>(row + i);
+      const bool is_q = i < qw;
+      const int wi = is_q ? i : i - qw;
+      const float* wn = is_q ? q_norm : k_norm;
+      f32x4 w = {1.f, 1.f, 1.f, 1.f};
+      if (wn != nullptr) w = *reinterpret_cast<const f32x4*>(wn + wi);
+      const float r = is_q ? rq : rk;
+      F o;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const T e = Elem<T>::st(get(f, j) * r * w[j]);
+        if constexpr (sizeof(T) == 2) o[j] = static_cast<short>(e); else o[j] = e;
+      }
+      if (is_q) {
+        *reinterpret_cast<F*>(q_out + static_cast<size_t>(t) * qw + i) = o;
+      } else if (kv_ok) {
+        const int g = wi / dim, fd = wi - g * dim;
+        T* slab = k_cache + (static_cast<size_t>(blk) * n_kv + g) * BS * dim;
+        *reinterpret_cast<F*>(slab + (static_cast<size_t>(fd >> 2) * BS + off) * 4) = o;
+      }
+    }
+  }
+  if constexpr (TPB == 4) {
+    const int t0 = blockIdx.x * 4;
+    bool group = t0 + 3 < n_tokens;   // (uniform over the workgroup)
+    if (group) {
+      const int s0 = slots[t0];
+      group = s0 >= 0 && (s0 & 3) == 0 && s0 / BS < num_blocks && slots[t0 + 1] == s0 + 1 && slots[t0 + 2] == s0 + 2 && slots[t0 + 3] == s0 + 3;
+    }
+    if (group) {   // a 4-key group of one page: one 4-key vector per value feature
+      const int s0 = slots[t0], b0 = s0 / BS, o0 = s0 - b0 * BS;
+      const T* v0 = qkv + static_cast<size_t>(t0) * row_stride + v_off;
+      for (int idx = threadIdx.x; idx < vw; idx += NT) {
+        const int g = idx / vdim, e = idx - g * vdim;
+        F o;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const T x = v0[static_cast<size_t>(j) * row_stride + idx];
+          if constexpr (sizeof(T) == 2) o[j] = static_cast<short>(x); else o[j] = x;
+        }
+        T* slab = v_cache + (static_cast<size_t>(b0) * n_kv + g) * vdim * BS;
+        *reinterpret_cast<F*>(slab + (static_cast<size_t>(o0 >> 2) * vdim + e) * 4) = o;
+      }
+      return;
+    }
+  }
+  if (kv_ok) {
+    for (int idx = tid; idx < vw; idx += TPT) {
+      const int g = idx / vdim, e = idx - g * vdim;
+      T* slab = v_cache + (static_cast<size_t>(blk) * n_kv + g) * vdim * BS;
+      slab[(static_cast<size_t>(off >> 2) * vdim + e) * 4 + (off & 3)] = row[v_off + idx];
     }
   }
 }
@@ -712,19 +828,36 @@ BCG_API int bcg_short_conv(const void* y, int64_t y_stride, int C, const void* w
 BCG_API int bcg_rope_pairs_kv_write(const void* qkv, int64_t row_stride, const void* positions, const void* slots,
                                     const void* q_norm, const void* k_norm, float eps, const void* inv_freq, int half,
                                     const void* v_inv_freq, void* q_out, void* k_cache, void* v_cache, int T_, int n_q,
-                                    int n_kv, int dim, int vdim, int BS, int num_blocks, int is_f32, void* stream) {
+                                    int n_kv, int dim, int vdim, int v_off, float temp_coef, int temp_every, int BS,
+                                    int num_blocks, int is_f32, void* stream) {
   if (T_ <= 0) return 0;
+  if (v_off < 0 || temp_every < 0 || BS % 16) return -2;
   if (2 * half > dim || (half > 0 && (dim & 1)) || (v_inv_freq != nullptr && (vdim & 1))) return -2;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int *ps = static_cast<const int*>(positions), *sl = static_cast<const int*>(slots);
   const float *qn = static_cast<const float*>(q_norm), *kn = static_cast<const float*>(k_norm),
               *fr = static_cast<const float*>(inv_freq), *vf = static_cast<const float*>(v_inv_freq);
+  auto al = [](const void* q, int b) { return (reinterpret_cast<uintptr_t>(q) & (b - 1)) == 0; };
+  if (half == 0 && vf == nullptr && dim % 4 == 0 && vdim % 4 == 0 && row_stride % 4 == 0 && al(qkv, is_f32 ? 16 : 8) && al(q_out, 16) &&
+      al(k_cache, 16) && al(v_cache, 16) && al(qn, 16) && al(kn, 16)) {
+#define BCG_NORM_KV(TYPE, TPB)                                                                                                    \
+  norm_kv_kernel<TYPE, TPB><<<(T_ + TPB - 1) / TPB, NT, 0, s>>>(static_cast<const TYPE*>(qkv), row_stride, ps, sl, qn, kn, eps,  \
+                                                                static_cast<TYPE*>(q_out), static_cast<TYPE*>(k_cache),          \
+                                                                static_cast<TYPE*>(v_cache), n_q, n_kv, dim, vdim, v_off,        \
+                                                                temp_coef, temp_every, BS, num_blocks, T_)
+    if (T_ >= 1024) BCG_BY_TYPE((BCG_NORM_KV(float, 4)), (BCG_NORM_KV(bf16_t, 4)));
+    else BCG_BY_TYPE((BCG_NORM_KV(float, 1)), (BCG_NORM_KV(bf16_t, 1)));
+#undef BCG_NORM_KV
+    return BCG_CHECK_LAUNCH();
+  }
   BCG_BY_TYPE((rope_pairs_kv_kernel<float><<<T_, NT, 0, s>>>(static_cast<const float*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half,
                                                             vf, static_cast<float*>(q_out), static_cast<float*>(k_cache),
-                                                            static_cast<float*>(v_cache), n_q, n_kv, dim, vdim, BS, num_blocks)),
+                                                            static_cast<float*>(v_cache), n_q, n_kv, dim, vdim, v_off, temp_coef, temp_every, BS,
+                                                            num_blocks)),
               (rope_pairs_kv_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const bf16_t*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half,
                                                              vf, static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache),
-                                                             static_cast<bf16_t*>(v_cache), n_q, n_kv, dim, vdim, BS, num_blocks)));
+                                                             static_cast<bf16_t*>(v_cache), n_q, n_kv, dim, vdim, v_off, temp_coef, temp_every, BS,
+                                                             num_blocks)));
   return BCG_CHECK_LAUNCH();
 }
 
