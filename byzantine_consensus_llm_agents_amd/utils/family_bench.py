@@ -1,4 +1,4 @@
-"""Prefill / decode throughput of the Mofidra, Padadra, Mabivik and Sitidra families beside the Qwen3-style decoder
+"""Prefill / decode throughput of the Mofidra, Padadra, Mabivik, Sitidra and Sadodra families beside the Qwen3-style decoder
 at equal layer sizes (random weights, synthetic tokens), and the hot kernels against their
 rooflines.  ``bench.py --family-compare`` prints the result as one JSON line.
 
@@ -32,6 +32,14 @@ with the normaliser); every feed-forward routes top-2 of 8 gated experts of ff/4
 inside 2 of 4 groups, plus a shared expert of ff/2.  Its closest relative is Mabivik (fp32
 stream, masked attention beside recurrences on the same scan kernel, the same gated experts).
 
+Sadodra at equal size: the same width, query / KV head counts and feed-forward width (gated gelu:
+three matrices, as the decoder's); four layers (attention, latent attention, attention, a second
+latent attention that reads the first one's latents); the attention has 128 features per head
+(values are the keys), a 512-key window, capped and distance-biased scores; the latent attention 128
+query / key and 128 value features per head, a 128-wide latent (a cached row of 128 features, ONE KV
+head) and no window.  Its closest relatives are Mabivik (latent attention, post norms on an fp32
+stream), Padadra (windowed attention with whole-projection norms) and Mofidra (dense gelu).
+
 Rooflines: 2.5 PFLOP/s dense bf16 MFMA, 8 TB/s HBM.  A kernel's ``roof_frac`` is
 max(flops / peak, bytes / bandwidth) / measured time.  The recurrence runs on the vector ALUs:
 its compute roof is 157 TFLOP/s fp32.
@@ -42,13 +50,15 @@ import time
 
 import torch
 
-from ..models.config import MabivikConfig, MofidraConfig, ModelConfig, PadadraConfig, SitidraConfig
+from ..models.config import MabivikConfig, MofidraConfig, ModelConfig, PadadraConfig, SadodraConfig, SitidraConfig
 from ..models.mabivik import MabivikModel
 from ..models.mofidra import MofidraModel
 from ..models.padadra import PadadraModel
+from ..models.sadodra import SadodraModel
 from ..models.sitidra import SitidraModel
 from ..models.transformer import AttnMeta, DecoderModel
 from ..ops import get_ops
+from ..ops.reference import alibi_slopes
 
 PEAK_FLOPS, PEAK_BW = 2.5e15, 8.0e12
 PEAK_VALU = 157e12
@@ -115,6 +125,19 @@ def sitidra_config(s) -> SitidraConfig:
               for i in range(s["layers"])]
     return SitidraConfig.from_dict({"architecture": "Sitidra", "width": W, "vocab": s["vocab"], "norm": {"eps": 1e-5},
                                     "streams": 4, "logit_softcap": 50.0, "layers": layers}, "sitidra-bench")
+
+
+def sadodra_config(s) -> SadodraConfig:
+    H, G, W = s["heads"], s["kv_heads"], s["width"]
+    att = {"heads": H, "kv_heads": G, "dim": 128, "vdim": 128, "scale": 0.088, "softcap": 30.0, "mask": {"size": 512},
+           "q_temp": {"coef": 0.1, "every": 256}}
+    lat = {"heads": H, "dim": 128, "vdim": 128, "kv_rank": 128, "scale": 0.088}
+    layers = []
+    for i in range(s["layers"]):
+        mixer = att if i % 2 == 0 else (lat if i % 4 == 1 else dict(lat, kv_from=i - 2))
+        layers.append({"type": "attention" if i % 2 == 0 else "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": s["ff"]}})
+    return SadodraConfig.from_dict({"architecture": "Sadodra", "width": W, "vocab": s["vocab"], "max_positions": 8192,
+                                    "norm": {"eps": 1e-5}, "layers": layers}, "sadodra-bench")
 
 
 def decoder_config(s) -> ModelConfig:
@@ -614,6 +637,103 @@ def hyper_kernels(s, dev):
     return out
 
 
+def biased_kernels(s, dev):
+    """Sadodra's kernels beside the like kernels of Padadra, Mabivik and Mofidra at the same shapes."""
+    ops = get_ops("hip")
+    H, G, W, ff = s["heads"], s["kv_heads"], s["width"], s["ff"]
+    bf = torch.bfloat16
+    out = {}
+    n, ctx, window = 8, 1024, 512
+    T, b = n * ctx, 64
+    meta, nb = step_meta(n, ctx, ctx, 64, dev, True)
+    dmeta, nbd = step_meta(b, ctx, 1, 64, dev, True)
+    nb = max(nb, nbd)
+    pairs_w, pairs = sum(min(i + 1, window) for i in range(ctx)) * n, ctx * (ctx + 1) // 2 * n
+    slopes = alibi_slopes(H, dev)
+    sink = torch.randn(H, device=dev)
+
+    def entry(name, **fracs):
+        out[name] = {}
+        for family, (t, flops, io) in fracs.items():
+            out[name][family + "_ms"] = round(t * 1e3, 4)
+            out[name][family + "_roof_frac"] = _roof(flops, io, t)
+    # ---- windowed attention: capped and biased scores against a sink, one kernel otherwise ----
+    kc, vc = torch.randn(nb, G, BS, 128, device=dev, dtype=bf), torch.randn(nb, G, 128, BS, device=dev, dtype=bf)
+    for name, rows, m_, timer in (("prefill_attention", T, meta, _time), ("decode_attention", b, dmeta, _graph_time)):
+        q = torch.randn(rows, H, 128, device=dev, dtype=bf)
+        np_, io = (pairs_w, T * (H + G) * 256 * 2) if rows == T else (b * window, b * window * G * 256 * 2)
+        args = (m_, 0.088, 1, 0.0, -1.0, 1.0, 128, window)
+        entry(name, sadodra=(timer(lambda: ops.multimap_attention(q, kc, vc, *args, None, 0, 30.0, slopes)), 2 * H * 256 * np_, io),
+              padadra=(timer(lambda: ops.multimap_attention(q, kc, vc, *args, sink)), 2 * H * 256 * np_, io))
+    # ---- latent attention: 128-wide rows, all keys, against 192-wide rows and a window ----
+    for name, rows, m_, timer in (("prefill_latent_attention", T, meta, _time), ("decode_latent_attention", b, dmeta, _graph_time)):
+        res = {}
+        for family, kd, win in (("sadodra", 128, 0), ("mabivik", 192, window)):
+            q = torch.randn(rows, H, kd, device=dev, dtype=bf)
+            kl, vl = torch.randn(nb, 1, BS, kd, device=dev, dtype=bf), torch.randn(nb, 1, 128, BS, device=dev, dtype=bf)
+            keys = win or ctx
+            np_ = (pairs_w if win else pairs) if rows == T else b * keys
+            io = T * (H + 1) * (kd + 128) * 2 if rows == T else b * keys * (kd + 128) * 2
+            t = timer(lambda: ops.multimap_attention(q, kl, vl, m_, 0.088, 1, 0.0, -1.0, 1.0, 128, win, None))
+            res[family] = (t, 2 * H * (kd + 128) * np_, io)
+        entry(name, **res)
+    # ---- residual update, 8192 and 64 rows: layer norm of the sublayer's output + rounded copy ----
+    w1, b1, w2, b2 = (torch.randn(W, device=dev) for _ in range(4))
+    for rows, timer in ((T, _time), (b, _graph_time)):
+        x32, a = torch.randn(rows, W, device=dev), torch.randn(rows, W, device=dev, dtype=bf)
+        io = rows * W * (4 + 4 + 2 + 2)
+        it = dict(iters=20) if rows == T else dict(iters=50)
+        entry(f"residual_norm_{rows}_rows",
+              sadodra=(timer(lambda: ops.residual_post_norm(x32, a, ("ln", w1, b1, 1e-5), ("copy",), bf), **it), 0, io),
+              mabivik=(timer(lambda: ops.residual_post_norm(x32, a, ("dyt", 0.5, w1, b1), ("dyt", 0.7, w2, b2), bf), **it), 0, io),
+              mofidra=(timer(lambda: ops.residual_add_rmsnorm32(x32, [a], w1, 1e-5, 1.0, bf), **it), 0, io))
+        if rows == T:
+            entry("residual_norm_final", sadodra=(timer(lambda: ops.residual_post_norm(x32, a, ("ln", w1, b1, 1e-5), ("ln", w2, b2, 1e-5), bf), **it), 0, io))
+    # ---- embedding ----
+    table, ptab = torch.randn(s["vocab"], W, device=dev, dtype=bf), torch.randn(8192, W, device=dev, dtype=bf)
+    tok = torch.randint(0, s["vocab"], (T,), dtype=torch.int32, device=dev)
+    entry("embedding", sadodra=(_time(lambda: ops.embed_position(tok, meta.positions, table, ptab, bf), iters=20), 0, T * W * (2 + 4 + 2) + ctx * W * 2),
+          mabivik=(_time(lambda: ops.embed_scale_dyt(tok, table, 1.0, (0.5, w1, b1), bf), iters=20), 0, T * W * (2 + 4 + 2)))
+    # ---- cache writes ----
+    width = (H + G) * 128
+    qn, kn = torch.ones(H * 128, device=dev), torch.ones(G * 128, device=dev)
+    inv, vinv, none = torch.rand(32, device=dev), torch.rand(64, device=dev), torch.empty(0, device=dev)
+    for name, rows, m_ in (("cache_write", T, meta), ("cache_write_decode", b, dmeta)):
+        y = torch.randn(rows, width + G * 128, device=dev, dtype=bf)
+        yk = y[:, :width].contiguous()
+        entry(name, sadodra=(_graph_time(lambda: ops.rope_pairs_kv_write(yk, m_.positions, m_.slots, H, G, 128, 128, qn, kn, 1e-5, none, None,
+                                                                         kc, vc, True, (0.1, 256)), iters=50), 0, rows * (2 * width + G * 128) * 2),
+              padadra=(_graph_time(lambda: ops.rope_pairs_kv_write(y, m_.positions, m_.slots, H, G, 128, 128, qn, kn, 1e-5, inv, vinv, kc, vc),
+                                   iters=50), 0, rows * (width + G * 128) * 2 * 2))
+        res = {}
+        for family, rd in (("sadodra", 0), ("mabivik", 64)):
+            kl, vl = torch.randn(nb, 1, BS, 128 + rd, device=dev, dtype=bf), torch.randn(nb, 1, 128, BS, device=dev, dtype=bf)
+            fr = torch.rand(rd // 2, device=dev)
+            yl = torch.randn(rows, H * 128 + 128 + rd + H, device=dev, dtype=bf)
+            t = _graph_time(lambda: ops.latent_kv_write(yl, H * 128, 128, rd, qn[:128], 1e-5, m_.positions, m_.slots, fr, 1.0, kl, vl), iters=50)
+            res[family] = (t, 0, rows * (2 * (128 + rd) + 128) * 2)
+        entry("latent_" + name, **res)
+    # ---- the latent's per-head products, the gate, the feed-forward's activation ----
+    for name, rows, timer in (("head_products", T, _time), ("head_products_decode", b, _graph_time)):
+        y = torch.randn(rows, H * 128 + 128 + H, device=dev, dtype=bf)
+        q3, wk = y[:, :H * 128].view(rows, H, 128), torch.randn(H, 128, 128, device=dev, dtype=bf)
+        dst = torch.empty(rows, H, 128, device=dev, dtype=bf)
+        dst2 = torch.empty(rows, H, 192, device=dev, dtype=bf)
+        y2 = torch.randn(rows, H, 192, device=dev, dtype=bf)
+        fl, io = 2 * rows * H * 128 * 128, rows * H * 256 * 2 + H * 128 * 128 * 2
+        entry(name, sadodra=(timer(lambda: ops.head_linear(q3, wk, dst)), fl, io),
+              mabivik=(timer(lambda: ops.head_linear(y2[:, :, :128], wk, dst2[:, :, :128])), fl, io))
+    att, gh, gf = torch.randn(T, H * 128, device=dev, dtype=bf), torch.randn(T, H, device=dev, dtype=bf), torch.randn(T, H * 128, device=dev, dtype=bf)
+    entry("output_gate", sadodra=(_time(lambda: ops.gate_mul(att, gh, "sigmoid", 128), iters=20), 0, T * H * 128 * 4),
+          mabivik=(_time(lambda: ops.gate_mul(att, gf, "sigmoid"), iters=20), 0, T * H * 128 * 6))
+    for rows, timer in ((T, _time), (b, _graph_time)):
+        both, one = torch.randn(rows, 2 * ff, device=dev, dtype=bf), torch.randn(rows, ff, device=dev, dtype=bf)
+        entry(f"activation_{rows}_rows", sadodra=(timer(lambda: ops.gated_act(both, "gelu_tanh")), 0, rows * ff * 6),
+              mofidra=(timer(lambda: ops.act_fn(one, "gelu_tanh")), 0, rows * ff * 4),
+              decoder=(timer(lambda: ops.silu_mul(both)), 0, rows * ff * 6))
+    return out
+
+
 def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
     dev = torch.device("cuda", torch.cuda.current_device())
     ops = get_ops("hip")
@@ -628,6 +748,7 @@ def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
                                  ("padadra", lambda: PadadraModel(padadra_config(s), ops, dev)),
                                  ("mabivik", lambda: MabivikModel(mabivik_config(s), ops, dev)),
                                  ("sitidra", lambda: SitidraModel(sitidra_config(s), ops, dev)),
+                                 ("sadodra", lambda: SadodraModel(sadodra_config(s), ops, dev)),
                                  ("decoder", lambda: DecoderModel(decoder_config(s), ops, dev))):
                 if families and label.split("_")[0] not in families:
                     continue
@@ -637,7 +758,8 @@ def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
                 del model
                 torch.cuda.empty_cache()
             groups = (("mofidra", "kernels", kernel_pairs), ("padadra", "state_kernels", state_kernels),
-                      ("mabivik", "latent_kernels", latent_kernels), ("sitidra", "hyper_kernels", hyper_kernels))
+                      ("mabivik", "latent_kernels", latent_kernels), ("sitidra", "hyper_kernels", hyper_kernels),
+                      ("sadodra", "biased_kernels", biased_kernels))
             for family, key, fn in groups if kernels else ():
                 if not families or family in families:
                     entry[key] = fn(s, dev)

@@ -103,6 +103,19 @@ def test_gated_act(dtype, kind):
 
 
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
+@pytest.mark.parametrize("kind", ["sigmoid", "silu"])
+def test_gates_per_head_and_per_feature(dtype, kind):
+    """On and off the 4-column grid; the gate a column range of a wider row at aligned and odd offsets."""
+    ops = K.Env("hip", "cuda").ops
+    for rows, heads, vd, off, pad in ((5, 3, 20, 4, 8), (9, 5, 7, 3, 1), (130, 16, 128, 8, 0), (70001, 2, 4, 1, 3)):
+        x = torch.randn(rows, heads * vd).to(dtype).to(DEV)
+        for group in (vd, 1):
+            w = heads * vd // group
+            gate = (torch.randn(rows, off + w + pad) * 2).to(dtype).to(DEV)[:, off:off + w]
+            torch.testing.assert_close(ops.gate_mul(x, gate, kind, group).float(), ref.gate_mul(x, gate, kind, group).float(), **_tol(dtype))
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
 @pytest.mark.parametrize("H,G,d,pad", [(4, 2, 16, 4), (3, 3, 10, 3), (2, 1, 72, 0), (6, 2, 20, 8), (5, 1, 7, 1), (8, 2, 128, 16)])
 def test_keys_as_values_norms_and_temperature(dtype, H, G, d, pad):
     """The write without rotation: element and 4-feature forms, small and large steps; slots of large
