@@ -17,6 +17,9 @@ def model_class(family: str):
     if family == "sadodra":
         from .sadodra import SadodraModel
         return SadodraModel
+    if family == "vagozen":
+        from .vagozen import VagozenModel
+        return VagozenModel
     from .transformer import DecoderModel
     return DecoderModel
 

@@ -91,12 +91,20 @@ class MixerSpec:
 @dataclass(frozen=True)
 class FeedForwardSpec:
     """kind "dense": one ``ff``-wide layer.  kind "moe": ``experts`` layers of width ``ff`` of
-    which a token uses ``top``, plus an always-on gated expert of width ``shared_ff`` (0 = none)."""
+    which a token uses ``top``, plus an always-on gated expert of width ``shared_ff`` (0 = none).
+    ``limit`` > 0: the clamp of a clamped gated unit."""
     kind: str
     ff: int
     experts: int = 0
     top: int = 0
     shared_ff: int = 0
+    limit: float = 0.0
+
+
+def loop_runs(n: int, start: int, stop: int, times: int) -> tuple:
+    """Layer index of every layer run of ``n`` layers, in execution order: the span ``start ..
+    stop - 1`` repeats ``times`` times with the same weights."""
+    return tuple(range(start)) + tuple(range(start, stop)) * times + tuple(range(stop, n))
 
 
 @dataclass(frozen=True)
@@ -185,9 +193,7 @@ class MofidraConfig:
     def layer_runs(self) -> tuple:
         """Layer index of every layer run, in execution order: the loop span repeats
         ``loop_times`` times with the same weights; every run keeps a KV cache of its own."""
-        n = len(self.layers)
-        span = tuple(range(self.loop_start, self.loop_stop))
-        return tuple(range(self.loop_start)) + span * self.loop_times + tuple(range(self.loop_stop, n))
+        return loop_runs(len(self.layers), self.loop_start, self.loop_stop, self.loop_times)
 
     @property
     def num_layers(self) -> int:
@@ -388,7 +394,8 @@ class LatentAttentionSpec:
     = (factor, original, fast, slow) ramps the frequencies between two turn counts and multiplies
     cos and sin by ``0.1 ln(factor) + 1``.  ``window`` keys are visible (0 = all); ``kv_from``: the
     layer whose cache this one reads instead of holding one (-1 = its own); ``head_gate``: one sigmoid
-    output gate per head instead of one per value feature."""
+    output gate per head instead of one per value feature; ``gated`` False: no output gate;
+    ``rot_pairs``: features 2i and 2i + 1 turn together instead of i and i + rot_dims / 2."""
     heads: int
     dim: int
     rot_dim: int
@@ -402,6 +409,8 @@ class LatentAttentionSpec:
     rot_scaling: Optional[tuple] = None
     kv_from: int = -1
     head_gate: bool = False
+    gated: bool = True
+    rot_pairs: bool = False
 
     @property
     def q_width(self) -> int:
@@ -414,6 +423,8 @@ class LatentAttentionSpec:
 
     @property
     def gate_width(self) -> int:
+        if not self.gated:
+            return 0
         return self.heads if self.head_gate else self.heads * self.vdim
 
 
@@ -866,10 +877,208 @@ class SadodraConfig:
         return n
 
 
+@dataclass(frozen=True)
+class WindowAttentionSpec:
+    """GQA softmax attention with biased q / k / v projections over a sliding window of ``window`` keys (0 =
+    all) that keeps the sequence's first ``keep`` keys in sight at their true positions; interleaved-pair
+    rotary on the first ``rot_dims`` features of every q / k head, frequencies and amplitude scaled by
+    ``rot_scaling`` = (factor, original, fast, slow) as in `LatentAttentionSpec`."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int = 0
+    keep: int = 0
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: Optional[tuple] = None
+
+    @property
+    def q_width(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def k_width(self) -> int:
+        return self.kv_heads * self.dim
+
+    @property
+    def v_width(self) -> int:
+        return self.kv_heads * self.vdim
+
+
+@dataclass(frozen=True)
+class RetentionSpec:
+    """Linear attention with one fixed ``decay`` per head (state ``dim x vdim`` per head), rotate-half rotary on
+    the first ``rot_dims`` features of every q / k head, a full-width silu output gate behind unit-RMS heads."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: Optional[tuple] = None
+
+    @property
+    def qk_width(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def v_width(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class VagozenLayer:
+    type: str                    # "attention" | "retention" | "latent_attention"
+    mixer: object                # WindowAttentionSpec | RetentionSpec | LatentAttentionSpec
+    mlp: Optional[FeedForwardSpec]
+
+
+_RAMP = ("factor", "original", "fast", "slow")
+
+
+@dataclass(frozen=True)
+class VagozenConfig:
+    """Vagozen: RMS norms before and after every sublayer, a learned scale per feature on its normed
+    output, a weight-shared loop over a span of layers whose passes take the embedding in again and a
+    learned vector each, mixers of three kinds (windowed attention with kept first keys, retention, latent
+    attention) in the order the config lists, clamped gated feed-forwards (dense or routed), the embedding
+    table as output head.  Everything is read from the model directory's config.json."""
+    name: str
+    hidden_size: int
+    vocab_size: int
+    layers: tuple
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 1
+    rms_eps: float = 1e-6
+    logit_scale: float = 1.0
+    family: str = "vagozen"
+    max_position: int = 1 << 20
+    tie_embeddings: bool = True
+
+    @staticmethod
+    def _rot(m: dict, width: int) -> dict:
+        rot = m.get("rot") or {}
+        sc = rot.get("scaling")
+        out = dict(rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
+                   rot_scaling=tuple(float(sc[k]) for k in _RAMP) if sc else None)
+        if out["rot_dims"] < 0 or out["rot_dims"] % 2 or out["rot_dims"] > width:
+            raise ValueError("Vagozen: rot.dims even and not wider than what it turns")
+        return out
+
+    @classmethod
+    def _mixer(cls, kind: str, m: dict):
+        H, dim, vdim = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+        if kind == "attention":
+            mask = m.get("mask") or {}
+            spec = WindowAttentionSpec(heads=H, kv_heads=int(m.get("kv_heads") or H), dim=dim, vdim=vdim, scale=float(m["scale"]),
+                                       window=int(mask.get("size", 0)), keep=int(mask.get("keep_first", 0)), **cls._rot(m, dim))
+            if H % spec.kv_heads or spec.window < 0 or spec.keep < 0:
+                raise ValueError("Vagozen: heads must be a multiple of kv_heads, mask.size and mask.keep_first not negative")
+            return spec
+        if kind == "retention":
+            decay = tuple(float(d) for d in m["decay"])
+            if len(decay) != H:
+                raise ValueError("Vagozen: one decay per retention head")
+            return RetentionSpec(heads=H, dim=dim, vdim=vdim, decay=decay, **cls._rot(m, dim))
+        if kind == "latent_attention":
+            rot_dim = int(m.get("rot_dim", 0))
+            return LatentAttentionSpec(heads=H, dim=dim, rot_dim=rot_dim, vdim=vdim, q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]),
+                                       scale=float(m["scale"]), gated=False, rot_pairs=True, **cls._rot(m, rot_dim))
+        raise ValueError(f"Vagozen: unknown layer type {kind!r}")
+
+    @staticmethod
+    def _mlp(f: Optional[dict]) -> Optional[FeedForwardSpec]:
+        if f is None:
+            return None
+        if f["kind"] == "dense":
+            spec = FeedForwardSpec("dense", int(f["ff"]), limit=float(f["limit"]))
+        elif f["kind"] == "moe":
+            e, r = f["expert"], f["router"]
+            spec = FeedForwardSpec("moe", int(e["ff"]), int(r["experts"]), int(r["top"]), limit=float(e["limit"]))
+            if not 1 <= spec.top <= spec.experts:
+                raise ValueError("Vagozen: router.top must be in [1, experts]")
+        else:
+            raise ValueError(f"Vagozen: unknown feed-forward kind {f['kind']!r}")
+        if not spec.limit > 0:
+            raise ValueError("Vagozen: limit must be positive")
+        return spec
+
+    @classmethod
+    def from_dict(cls, c: dict, name: str = "vagozen") -> "VagozenConfig":
+        layers = tuple(VagozenLayer(e["type"], cls._mixer(e["type"], e["mixer"]), cls._mlp(e.get("mlp"))) for e in c["layers"])
+        loop = c.get("loop") or {}
+        start, stop, times = int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1))
+        if not 0 <= start <= max(start, stop) <= len(layers) or times < 1:
+            raise ValueError("Vagozen: loop span outside the layer list")
+        return cls(name=name, hidden_size=int(c["width"]), vocab_size=int(c["vocab"]), layers=layers, loop_start=start,
+                   loop_stop=max(start, stop), loop_times=times, rms_eps=float(c["norm"]["eps"]),
+                   logit_scale=float(c.get("logit_scale", 1.0)))
+
+    def to_dict(self) -> dict:
+        """The config.json form (inverse of `from_dict`)."""
+        out = []
+        for l in self.layers:
+            m, f = l.mixer, l.mlp
+            mixer = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim, "rot": {"dims": m.rot_dims, "base": m.rot_base}}
+            if m.rot_scaling:
+                mixer["rot"]["scaling"] = dict(zip(_RAMP, m.rot_scaling))
+            if l.type == "attention":
+                mixer.update(kv_heads=m.kv_heads, scale=m.scale)
+                if m.window:
+                    mixer["mask"] = {"size": m.window, "keep_first": m.keep}
+            elif l.type == "retention":
+                mixer["decay"] = list(m.decay)
+            else:
+                mixer.update(rot_dim=m.rot_dim, q_rank=m.q_rank, kv_rank=m.kv_rank, scale=m.scale)
+            mlp = None
+            if f is not None and f.kind == "dense":
+                mlp = {"kind": "dense", "ff": f.ff, "limit": f.limit}
+            elif f is not None:
+                mlp = {"kind": "moe", "expert": {"ff": f.ff, "limit": f.limit}, "router": {"experts": f.experts, "top": f.top}}
+            out.append({"type": l.type, "mixer": mixer, "mlp": mlp})
+        d = {"architecture": "Vagozen", "width": self.hidden_size, "vocab": self.vocab_size, "norm": {"eps": self.rms_eps},
+             "logit_scale": self.logit_scale, "layers": out}
+        if self.loop_stop > self.loop_start:
+            d["loop"] = {"start": self.loop_start, "stop": self.loop_stop, "times": self.loop_times}
+        return d
+
+    @property
+    def layer_runs(self) -> tuple:
+        """Layer index of every layer run, in execution order; every run keeps a cache or state of its own."""
+        return loop_runs(len(self.layers), self.loop_start, self.loop_stop, self.loop_times)
+
+    @property
+    def pass_starts(self) -> dict:
+        """Layer run that opens a pass of the loop -> number of the pass (empty without a loop)."""
+        span = self.loop_stop - self.loop_start
+        return {self.loop_start + t * span: t for t in range(self.loop_times)} if span > 0 else {}
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layer_runs)
+
+    def num_params(self) -> int:
+        W, n = self.hidden_size, self.vocab_size * self.hidden_size
+        for l in self.layers:
+            m, f = l.mixer, l.mlp
+            if l.type == "attention":
+                n += W * (m.q_width + m.k_width + m.v_width + m.heads * m.vdim)
+            elif l.type == "retention":
+                n += W * (2 * m.qk_width + 3 * m.v_width)
+            else:
+                n += W * (m.q_rank + m.key_width + m.heads * m.vdim) + m.q_rank * m.q_width + m.heads * m.kv_rank * (m.dim + m.vdim)
+            if f is not None:
+                n += 3 * W * f.ff * max(1, f.experts) + W * f.experts
+        return n
+
+
 # config.json "architecture" (lower case) -> configuration class; these families take token ids
 # when a checkpoint ships no tokenizer
 ARCHITECTURES = {"mofidra": MofidraConfig, "padadra": PadadraConfig, "mabivik": MabivikConfig, "sitidra": SitidraConfig,
-                 "sadodra": SadodraConfig}
+                 "sadodra": SadodraConfig, "vagozen": VagozenConfig}
 
 PRESETS = {
     "Qwen/Qwen3-8B": ModelConfig("Qwen/Qwen3-8B", "qwen3", 4096, 36, 32, 8, 128, 12288, 151936,

@@ -28,7 +28,7 @@ Kernel plan of one layer (HIP backend; the torch backend runs the same ops from
 ``ops/reference.py``):
 
     latent_attention  fused GEMM [dq | dkv | g] -> rmsnorm_cols (query latent) -> uq GEMM ->
-                      head_linear (W_uk^T q per head, straight into the packed query) + rope_half_tail;
+                      head_linear (W_uk^T q per head, straight into the packed query) + rope_tail;
                       latent_kv_write (norm, rotary, paged write) -> multimap_attention (one map,
                       one KV head, window) -> head_linear (W_uv) -> gate_mul -> o GEMM
     delta             fused GEMM [q | k | v | beta | a | g] -> short_conv (silu) -> delta_prepare ->

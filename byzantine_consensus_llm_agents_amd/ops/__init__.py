@@ -24,14 +24,14 @@ def _torch_ops() -> SimpleNamespace:
         return _ref.paged_attention(q, k_cache, v_cache, layer, block_tables, q_start, seq_lens, scale)
 
     def multimap_attention(q, k_cache, v_cache, meta, scale, maps, lam, head_eps, out_scale, vdim, window=0, sink=None,
-                           chunk=0, softcap=0.0, slopes=None):
+                           chunk=0, softcap=0.0, slopes=None, keep=0):
         # tiles / single-row lists only tell the HIP kernels how to walk the batch
         q_start = meta.q_start
         if q_start is None:  # decode: one row per sequence
             q_start = torch.arange(q.shape[0] + 1, dtype=torch.int32, device=q.device)
         lens = meta.seq_lens if meta.attn_seq_lens is None else meta.attn_seq_lens
         return _ref.multimap_attention(q, k_cache, v_cache, meta.block_tables, q_start, lens, scale, maps,
-                                       lam, head_eps, out_scale, vdim, window, sink, chunk, softcap, slopes)
+                                       lam, head_eps, out_scale, vdim, window, sink, chunk, softcap, slopes, keep)
 
     return SimpleNamespace(
         name="torch",
@@ -57,7 +57,7 @@ def _torch_ops() -> SimpleNamespace:
         residual_post_norm=_ref.residual_post_norm,
         rmsnorm_cols=_ref.rmsnorm_cols,
         latent_kv_write=_ref.latent_kv_write,
-        rope_half_tail=_ref.rope_half_tail,
+        rope_tail=_ref.rope_tail,
         head_linear=_ref.head_linear,
         gate_mul=_ref.gate_mul,
         ssm_prepare=_ref.ssm_prepare,
@@ -72,6 +72,7 @@ def _torch_ops() -> SimpleNamespace:
         moe_route_scored=_ref.moe_route_scored,
         softcap=_ref.softcap,
         embed_position=_ref.embed_position,
+        retention_prepare=_ref.retention_prepare,
         linear=torch.nn.functional.linear,
         rmsnorm=_ref.rmsnorm,
         add_rmsnorm=_ref.add_rmsnorm,

@@ -92,7 +92,7 @@ def load_library(path: str = None) -> ctypes.CDLL:
                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_gemm_tile": [c_int, ctypes.POINTER(c_int), ctypes.POINTER(c_int)],
         "bcg_gemm_num_cfgs": [],
-        "bcg_embed_scale_rmsnorm": [c_void_p, c_void_p, c_float, c_void_p, c_float, c_float, c_void_p, c_void_p,
+        "bcg_embed_scale_rmsnorm": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_float, c_float, c_void_p, c_void_p,
                                     c_int, c_int, c_int, c_int, c_void_p],
         "bcg_residual_add_rmsnorm32": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float,
                                        c_float, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -103,9 +103,13 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_multimap_attention": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                                    c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                    c_float, c_float, c_float, c_float, c_int, c_int, c_int, c_int, c_void_p, c_float,
-                                   c_void_p, c_void_p],
+                                   c_void_p, c_int, c_void_p],
         "bcg_embed_position": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                c_int, c_void_p],
+        "bcg_residual_rms_norm": [c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_int, c_int,
+                                  c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+        "bcg_retention_prepare": [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_float,
+                                  c_void_p, c_void_p, c_int, c_int, c_void_p],
         "bcg_residual_layer_norm": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_void_p,
                                     c_float, c_void_p, c_int, c_int, c_int, c_void_p],
         "bcg_embed_hashed_bigram": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
@@ -116,7 +120,7 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_short_conv": [c_void_p, c_int64, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                            c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
         "bcg_rope_pairs_kv_write": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int,
-                                    c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                    c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                     c_float, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_rotate_pairs": [c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_hgrn2_prepare": [c_void_p, c_int64, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
@@ -124,7 +128,8 @@ def load_library(path: str = None) -> ctypes.CDLL:
         "bcg_delta_prepare": [c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p,
                               c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_gated_state_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
-                                 c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                 c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                 c_void_p],
         "bcg_head_norm_gate": [c_void_p, c_void_p, c_float, c_void_p, c_int64, c_void_p, c_int, c_int, c_int, c_int, c_void_p,
                                c_int, c_int, c_void_p],
         "bcg_hyper_embed_norm": [c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int, c_int,
@@ -146,11 +151,11 @@ def load_library(path: str = None) -> ctypes.CDLL:
                                    c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
         "bcg_rmsnorm_cols": [c_void_p, c_int64, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p],
         "bcg_latent_kv_write": [c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
-                                c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
-        "bcg_rope_half_tail": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_int,
-                               c_int, c_int, c_void_p],
+                                c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+        "bcg_rope_tail": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_int, c_int,
+                          c_int, c_int, c_void_p],
         "bcg_gate_mul": [c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p],
-        "bcg_gated_act": [c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p],
+        "bcg_gated_act": [c_void_p, c_void_p, c_int64, c_int, c_int, c_float, c_int, c_void_p],
         "bcg_ssm_prepare": [c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_gated_group_norm": [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_float, c_void_p,
@@ -162,7 +167,7 @@ def load_library(path: str = None) -> ctypes.CDLL:
                           c_int, c_int, c_void_p],
         "bcg_moe_align": [c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p],
         "bcg_moe_gemm": [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_int, c_int,
-                         c_int, c_int, c_int, c_int, c_int, c_void_p],
+                         c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
         "bcg_moe_combine": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
         "bcg_guided_sample": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                               c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p,

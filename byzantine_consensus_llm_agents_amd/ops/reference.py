@@ -356,9 +356,12 @@ def rmsnorm32(x: torch.Tensor, w: torch.Tensor, eps: float, w_offset: float, out
     return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * (w_offset + w.float())).to(out_dtype)
 
 
-def embed_scale_rmsnorm(tokens, table, scale: float, w, eps: float, w_offset: float, out_dtype):
-    """(norm(scale * E[tokens]) in ``out_dtype``, scale * E[tokens] in fp32)."""
+def embed_scale_rmsnorm(tokens, table, scale: float, w, eps: float, w_offset: float, out_dtype, add=None):
+    """(norm of the stream in ``out_dtype``, fp32 stream ``scale * E[tokens]`` (+ ``add`` fp32 [W], one
+    vector for all rows))."""
     residual = table.index_select(0, tokens.long()).float() * scale
+    if add is not None:
+        residual = residual + add.float()
     return rmsnorm32(residual, w, eps, w_offset, out_dtype), residual
 
 
@@ -406,12 +409,13 @@ def rope_multi_kv_write(qkv, positions, slots, n_q: int, n_kv: int, maps: int, d
 
 def multimap_attention(q, k_cache, v_cache, block_tables, q_start, seq_lens, scale: float, maps: int,
                        lam: float, head_eps: float, out_scale: float, vdim: int, window: int = 0, sink=None,
-                       chunk: int = 0, softcap: float = 0.0, slopes=None):
+                       chunk: int = 0, softcap: float = 0.0, slopes=None, keep: int = 0):
     """Causal GQA attention with ``maps`` softmax maps per head over shared values:
     ``o = a_0 - lam * a_1`` (maps = 2; maps = 1: ``a_0``), then per head
     ``o / sqrt(mean(o^2) + head_eps) * out_scale`` (``head_eps < 0``: only the scale).
     Sequence b's query rows ``q_start[b]:q_start[b+1]`` are its last positions.  ``window`` > 0:
-    position i sees only j with i - j < window.  ``chunk`` > 0: position i sees only j of its own
+    position i sees only j with i - j < window, and (``keep`` > 0) the first ``keep`` positions of the sequence.
+    ``chunk`` > 0: position i sees only j of its own
     chunk, floor(j / chunk) = floor(i / chunk), chunks counted from position 0.  ``sink`` fp32 [n_q]: the softmax denominator of
     head h also holds ``exp(sink[h])`` (no key, no value, not scaled).  ``softcap`` > 0: the scaled score s
     becomes ``softcap tanh(s / softcap)``; ``slopes`` fp32 [n_q]: then ``slopes[h] (i - j)`` is taken off.  Returns
@@ -437,7 +441,7 @@ def multimap_attention(q, k_cache, v_cache, block_tables, q_start, seq_lens, sca
         kpos = torch.arange(ctx, device=q.device)[None, :]
         hidden = kpos > qpos
         if window > 0:
-            hidden = hidden | (kpos < qpos - window + 1)
+            hidden = hidden | ((kpos < qpos - window + 1) & (kpos >= keep))
         if chunk > 0:
             hidden = hidden | (kpos < qpos - qpos % chunk)
         o = None
@@ -487,10 +491,10 @@ def moe_route(h, router_w, router_b, top: int, gate_w=None):
     return idx[:, :top].to(torch.int32), torch.softmax(val[:, :top], dim=-1), gate
 
 
-def moe_experts(h, up, down, idx, weights, kind: str = "relu2"):
+def moe_experts(h, up, down, idx, weights, kind: str = "relu2", limit: float = 0.0):
     """``sum_j weights[t, j] * down[e] act(up[e] h_t)``, e = idx[t, j]; up [E, ff, W],
     down [E, W, ff].  kind "silu_gated": up is [E, 2 ff, W], rows [gate; up], and the hidden
-    activation is ``silu(gate h) * (up h)``.  Hidden activations are rounded to the activation dtype like a
+    activation is ``silu(gate h) * (up h)``; kind "clamped_glu": the same rows, `clamped_glu` with ``limit``.  Hidden activations are rounded to the activation dtype like a
     projection's output; the weighted sum is returned in fp32 (it goes into the fp32 residual)."""
     T, W = h.shape
     out = torch.zeros(T, W, dtype=torch.float32, device=h.device)
@@ -503,6 +507,8 @@ def moe_experts(h, up, down, idx, weights, kind: str = "relu2"):
         if kind == "silu_gated":
             ff = z.shape[1] // 2
             hid = (act_fn(z[:, :ff], "silu").float() * z[:, ff:].float()).to(z.dtype)
+        elif kind == "clamped_glu":
+            hid = clamped_glu(z, limit)
         else:
             hid = act_fn(z, kind)
         y = torch.nn.functional.linear(hid, down[e])
@@ -625,10 +631,10 @@ def scaled_inv_freq(dims: int, base: float, scaling=None, device=None) -> torch.
     return f.float().to(device)
 
 
-def _turn_pairs(x, ang):
-    """x [..., 2n]: the pair (2i, 2i + 1) turned by ang[..., i]."""
+def _turn_pairs(x, ang, amp: float = 1.0):
+    """x [..., 2n]: the pair (2i, 2i + 1) turned by ang[..., i]; cos and sin times amp."""
     a, b = x[..., 0::2], x[..., 1::2]
-    c, s = ang.cos(), ang.sin()
+    c, s = ang.cos() * amp, ang.sin() * amp
     return torch.stack([a * c - b * s, b * c + a * s], dim=-1).flatten(-2)
 
 
@@ -639,10 +645,10 @@ def query_temperature(positions, coef: float, every: int):
 
 
 def rope_pairs_kv_write(qkv, positions, slots, n_q: int, n_kv: int, dim: int, vdim: int, q_norm, k_norm, eps: float,
-                        inv_freq, v_inv_freq, k_cache, v_cache, v_is_k: bool = False, q_temp=None):
+                        inv_freq, v_inv_freq, k_cache, v_cache, v_is_k: bool = False, q_temp=None, amp: float = 1.0):
     """Row ``[q | k | v | ...]``: one RMS norm over the whole q part (weight ``q_norm``
     [n_q dim]; None = no norm) and one over the whole k part, then every q / k head's features
-    (2i, 2i + 1), i < len(inv_freq), are turned by ``position * inv_freq[i]``; every v head's pairs
+    (2i, 2i + 1), i < len(inv_freq), are turned by ``position * inv_freq[i]``, cos and sin times ``amp``; every v head's pairs
     by ``position * v_inv_freq[i]`` (None: values as they are).  ``v_is_k``: the row is ``[q | k | ...]`` and the
     values are the k part as projected, before its norm.  ``q_temp`` = (coef, every): q at position p is
     multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)``.  K / V go to the paged cache of
@@ -663,8 +669,8 @@ def rope_pairs_kv_write(qkv, positions, slots, n_q: int, n_kv: int, dim: int, vd
     r = 2 * inv_freq.numel()
     if r:
         ang = pos * inv_freq.float()[None, None, :]
-        q = torch.cat([_turn_pairs(q[..., :r], ang), q[..., r:]], -1)
-        k = torch.cat([_turn_pairs(k[..., :r], ang), k[..., r:]], -1)
+        q = torch.cat([_turn_pairs(q[..., :r], ang, amp), q[..., r:]], -1)
+        k = torch.cat([_turn_pairs(k[..., :r], ang, amp), k[..., r:]], -1)
     if v_inv_freq is not None:
         v = _turn_pairs(v, pos * v_inv_freq.float()[None, None, :])
     bs = k_cache.shape[2]
@@ -720,13 +726,15 @@ def gated_state_scan(q, k, g, v, beta, meta, state, delta: bool, unit_last: bool
         S <- S + k_t u^T;   o_t = S^T q_t
 
     q / k [T, Gq, dim] fp32 (head h reads q / k head h // (H / Gq)), g fp32 [T, H, dim] (a decay
-    per key channel) or [T, H, 1] (one per head), v [T, H vdim], beta [T, H] fp32 or None;
+    per key channel), [T, H, 1] (one per head) or [H] (one per head, the same for every token), v [T, H vdim], beta [T, H] fp32 or None;
     ``state`` [rows, H, dim, vdim] fp32 is read (unless the segment starts at position 0) and left
     at the segment's last token.  ``unit_last`` (without the delta rule): v is [T, H (vdim - 1)] and the
     state's last column reads a value of 1 for every token, so it accumulates the written keys alone
     (a normaliser beside the memory); o's last column is then its product with q.  Returns fp32 o [T, H, vdim]."""
-    T, H = g.shape[:2]
-    vdim = state.shape[3]
+    T = q.shape[0]
+    if g.dim() == 1:
+        g = g.reshape(1, -1, 1).expand(T, -1, 1)
+    H, vdim = g.shape[1], state.shape[3]
     per = H // q.shape[1]
     if unit_last:
         vf = torch.cat([v.float().reshape(T, H, vdim - 1), torch.ones(T, H, 1, device=v.device)], -1)
@@ -757,13 +765,15 @@ def gated_state_scan(q, k, g, v, beta, meta, state, delta: bool, unit_last: bool
 
 def head_norm_gate(o, w, eps: float, gate, out_dtype, gate_act: str = "sigmoid", floor=None):
     """o fp32 [T, H, vdim]: every head divided by its root mean square, times ``w`` ([vdim], or
-    [H vdim]: a weight per head), times ``sigmoid(gate)`` or ``silu(gate)`` (gate [T, H vdim] logits or
+    [H vdim]: a weight per head; None: no weight), times ``sigmoid(gate)`` or ``silu(gate)`` (gate [T, H vdim] logits or
     None; ``gate_act``); returns [T, H vdim] in ``out_dtype``.  ``floor`` fp32 [T, H]: o has one more
     column, a normaliser, and the head is first divided by ``max(|normaliser|, floor) + 1e-6``."""
     if floor is not None:
         o = o[..., :-1] / (torch.maximum(o[..., -1].abs(), floor.float()) + 1e-6)[..., None]
     T, H, vdim = o.shape
-    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * w.float().reshape(-1, vdim)
+    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)
+    if w is not None:
+        y = y * w.float().reshape(-1, vdim)
     if gate is not None:
         z = gate.float().reshape(T, H, vdim)
         y = y * (torch.sigmoid(z) if gate_act == "sigmoid" else z * torch.sigmoid(z))
@@ -793,13 +803,21 @@ def embed_scale_dyt(tokens, table, scale: float, norm, out_dtype):
     return x, dyt(x, norm, out_dtype)
 
 
-def residual_post_norm(x, y, post, pre, out_dtype):
+def residual_post_norm(x, y, post, pre, out_dtype, entry=None):
     """``x += post(y)`` in fp32, in place, with ``post`` = ("dyt", alpha, w, b), ("rms", w, eps)
     (``y / sqrt(mean(y^2) + eps) * w``) or ("ln", w, b, eps) (`layer_norm32` of y); then returns what the
     next reader of x takes: ``pre`` = ("dyt", alpha, w, b) -> `dyt` of the new x, ("ln", w, b, eps) (with a
-    layer norm as ``post``) -> its layer norm, ("copy",) -> x rounded to ``out_dtype``, None -> None."""
-    yf = y.float()
-    if post[0] == "dyt":
+    layer norm as ``post``) -> its layer norm, ("rms", w, eps) (with an RMS norm as ``post``) -> its RMS norm,
+    ("copy",) -> x rounded to ``out_dtype``, None -> None.  ``entry`` = (vec, tokens, table) (RMS ``post``):
+    x also takes ``vec`` (fp32 [W]) and, with a table, the row ``table[token]``, behind the post norm
+    and before the next reader.  ``y`` None: no sublayer output (only ``entry`` and the next reader)."""
+    if y is None:
+        yf, post = None, ("none",)
+    else:
+        yf = y.float()
+    if post[0] == "none":
+        pass
+    elif post[0] == "dyt":
         x.add_(torch.tanh(float(post[1]) * yf) * post[2].float() + post[3].float())
     elif post[0] == "rms":
         x.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + float(post[2])) * post[1].float())
@@ -807,12 +825,17 @@ def residual_post_norm(x, y, post, pre, out_dtype):
         x.add_(layer_norm32(yf, post[1], float(post[3]), torch.float32, post[2]))
     else:
         raise ValueError(f"unknown post norm {post[0]!r}")
+    if entry is not None:
+        vec, tokens, table = entry
+        x.add_(vec.float() if table is None else table.index_select(0, tokens.long()).float() + vec.float())
     if pre is None:
         return None
     if pre[0] == "copy":
         return x.to(out_dtype)
     if pre[0] == "ln":
         return layer_norm32(x, pre[1], float(pre[3]), out_dtype, pre[2])
+    if pre[0] == "rms":
+        return rmsnorm32(x, pre[1], float(pre[2]), 0.0, out_dtype)
     return dyt(x, pre[1:], out_dtype)
 
 
@@ -854,24 +877,33 @@ def _turn_half(x, positions, inv_freq, amp: float):
     return torch.cat([a * c - b * s, b * c + a * s, x[..., 2 * half:]], dim=-1)
 
 
+def _turn_tail(x, positions, inv_freq, amp: float, pairs: bool):
+    """`_turn_half`, or (``pairs``) the same with neighbours: features 2i and 2i + 1 turn together."""
+    if not pairs or not inv_freq.numel():
+        return _turn_half(x, positions, inv_freq, amp)
+    r = 2 * inv_freq.numel()
+    ang = positions.float().reshape(-1, *([1] * (x.dim() - 1))) * inv_freq.float()
+    return torch.cat([_turn_pairs(x[..., :r], ang, amp), x[..., r:]], dim=-1)
+
+
 def latent_kv_write(y, off: int, kv_rank: int, rot_dim: int, w, eps: float, positions, slots, inv_freq, amp: float,
-                    k_cache, v_cache):
+                    k_cache, v_cache, pairs: bool = False):
     """Columns ``off : off + kv_rank`` of ``y`` are RMS-normed (weight ``w``) into the latent c,
-    the next ``rot_dim`` are turned by the position (`_turn_half`, not normed); the token's cache
+    the next ``rot_dim`` are turned by the position (`_turn_tail`, not normed); the token's cache
     row becomes K = [c | turned part], V^T = c."""
     c = rmsnorm_cols(y, off, kv_rank, w, eps, torch.float32)
-    kr = _turn_half(y[:, off + kv_rank:off + kv_rank + rot_dim].float(), positions, inv_freq, amp)
+    kr = _turn_tail(y[:, off + kv_rank:off + kv_rank + rot_dim].float(), positions, inv_freq, amp, pairs)
     bs = k_cache.shape[2]
     blk, o = (slots // bs).long(), (slots % bs).long()
     k_cache[blk, 0, o] = torch.cat([c, kr], -1).to(k_cache.dtype)
     v_cache[blk, 0, :, o] = c.to(v_cache.dtype)
 
 
-def rope_half_tail(src, src_off: int, dst, dst_off: int, positions, inv_freq, amp: float):
+def rope_tail(src, src_off: int, dst, dst_off: int, positions, inv_freq, amp: float, pairs: bool = False):
     """``dst[:, h, dst_off:] = turn(src[:, h, src_off:])`` for every head of src [T, H, Ds] / dst
     [T, H, Dd] (tails of equal width): the first ``2 len(inv_freq)`` features of the tail are turned
-    by the position (feature i pairs with i + half), the rest copied."""
-    dst[:, :, dst_off:] = _turn_half(src[:, :, src_off:].float(), positions, inv_freq, amp).to(dst.dtype)
+    by the position (feature i pairs with i + half, or with ``pairs`` feature 2i with 2i + 1), the rest copied."""
+    dst[:, :, dst_off:] = _turn_tail(src[:, :, src_off:].float(), positions, inv_freq, amp, pairs).to(dst.dtype)
     return dst
 
 
@@ -928,10 +960,20 @@ def gelu_gather_mul(z, tokens, table, off: int):
     return (act_fn(z.float(), "gelu_tanh") * e).to(z.dtype)
 
 
-def gated_act(both, kind: str = "silu"):
+def clamped_glu(both, limit: float):
+    """``g sigmoid(1.702 g) (u + 1)`` for a stacked [gate | up] projection [rows, 2 n], the gate clamped from
+    above and the up part from both sides at ``limit``; fp32 math, rounded once."""
+    n = both.shape[1] // 2
+    g, u = both[:, :n].float().clamp(max=limit), both[:, n:].float().clamp(-limit, limit)
+    return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(both.dtype)
+
+
+def gated_act(both, kind: str = "silu", limit: float = 0.0):
     """``act(both[:, :n]) * both[:, n:]`` for a stacked [gate | up] projection [rows, 2 n], act of
     `act_fn` ("silu" | "gelu_tanh"); the activation is rounded like a projection's output before the
-    product."""
+    product.  kind "clamped_glu": `clamped_glu` with ``limit``."""
+    if kind == "clamped_glu":
+        return clamped_glu(both, limit)
     n = both.shape[1] // 2
     return (act_fn(both[:, :n], kind).float() * both[:, n:].float()).to(both.dtype)
 
@@ -1074,3 +1116,16 @@ def alibi_slopes(heads: int, device=None) -> torch.Tensor:
     """fp32 [heads]: ``2^(-8 (h + 1) / heads)``, the distance slopes of biased attention heads."""
     h = torch.arange(heads, dtype=torch.float64)
     return torch.pow(2.0, -8.0 * (h + 1.0) / heads).float().to(device)
+
+
+# ------------------------------------------------------------------ retention (models/vagozen.py)
+
+def retention_prepare(y, off_q: int, off_k: int, heads: int, dim: int, k_scale: float, positions, inv_freq, amp: float = 1.0):
+    """The read and write vectors of a retention mixer from its fused projection: the columns
+    ``off_q : off_q + heads dim`` and ``off_k : ...`` of ``y``, every head turned by the position
+    (`_turn_half`), k then times ``k_scale``.  Returns fp32 (q, k), each [T, heads, dim]: with a decay
+    per head the operands of `gated_state_scan`."""
+    T, n = y.shape[0], heads * dim
+    q = _turn_half(y[:, off_q:off_q + n].float().reshape(T, heads, dim), positions, inv_freq, amp)
+    k = _turn_half(y[:, off_k:off_k + n].float().reshape(T, heads, dim), positions, inv_freq, amp) * k_scale
+    return q.contiguous(), k.contiguous()

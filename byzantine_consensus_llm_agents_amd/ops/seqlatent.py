@@ -53,11 +53,44 @@ def seqlatent_ops(lib):
                "residual_layer_norm")
         return out
 
-    def residual_post_norm(x, y, post, pre, out_dtype):
+    def _residual_rms_norm(x, y, post, pre, out_dtype, entry):
+        T, W = x.shape
+        _req(W <= MAX_LN_WIDTH, f"RMS-normed residual: width <= {MAX_LN_WIDTH}")
+        pw, eps = None, 0.0
+        if y is not None:
+            _f32(post[1], W, "norm weight")
+            pw, eps = _p(post[1]), float(post[2])
+        add = toks = table = None
+        vocab = 0
+        if entry is not None:
+            add, toks, table = entry
+            _f32(add, W, "entry vector")
+            if table is not None:
+                _i32(toks, T, "tokens")
+                _req(table.dim() == 2 and table.shape[1] == W and table.is_contiguous() and table.dtype == out_dtype,
+                     "entry table [vocab, W] in the activation dtype")
+                vocab = table.shape[0]
+        out, pre_kind, qw, pre_eps = None, 0, None, 0.0
+        if pre is not None:
+            out = torch.empty(T, W, dtype=out_dtype, device=x.device)
+            _req(pre[0] in ("copy", "rms"), "behind an RMS norm with an entry: a rounded copy or an RMS norm of the stream")
+            pre_kind = 1
+            if pre[0] == "rms":
+                _f32(pre[1], W, "norm weight")
+                pre_kind, qw, pre_eps = 2, _p(pre[1]), float(pre[2])
+        _check(lib.bcg_residual_rms_norm(_p(x), _p(y), int(y is not None and y.dtype == torch.float32), pw, eps, _p(add),
+                                         _p(toks) if table is not None else None, _p(table), vocab, pre_kind, qw, pre_eps,
+                                         _p(out), T, W, int(out_dtype == torch.float32), _stream()), "residual_rms_norm")
+        return out
+
+    def residual_post_norm(x, y, post, pre, out_dtype, entry=None):
         _req(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "residual fp32 [T, W]")
         T, W = x.shape
-        _req(y.shape == (T, W) and y.is_contiguous() and y.dtype in (out_dtype, torch.float32),
+        _req(y is None or (y.shape == (T, W) and y.is_contiguous() and y.dtype in (out_dtype, torch.float32)),
              "sublayer output [T, W] in the activation dtype or fp32")
+        if y is None or entry is not None or (post[0] == "rms" and pre is not None and pre[0] == "rms"):
+            _req(y is None or post[0] == "rms", "an entry into the stream: behind an RMS norm")
+            return _residual_rms_norm(x, y, post, pre, out_dtype, entry)
         if post[0] == "dyt":
             kind, (pa, pw, pb), eps = 0, _dyt(post[1:], W), 0.0
         elif post[0] == "rms":
@@ -87,7 +120,7 @@ def seqlatent_ops(lib):
         _check(lib.bcg_rmsnorm_cols(_p(y), y.stride(0), off, n, _p(w), eps, _p(out), T, _act(y), _stream()), "rmsnorm_cols")
         return out
 
-    def latent_kv_write(y, off, kv_rank, rot_dim, w, eps, positions, slots, inv_freq, amp, k_cache, v_cache):
+    def latent_kv_write(y, off, kv_rank, rot_dim, w, eps, positions, slots, inv_freq, amp, k_cache, v_cache, pairs=False):
         T = y.shape[0]
         _req(y.dim() == 2 and y.stride(1) == 1 and 0 <= off and off + kv_rank + rot_dim <= y.shape[1],
              "latent_kv_write: rows [T, >= off + kv_rank + rot_dim], unit column stride")
@@ -103,12 +136,12 @@ def seqlatent_ops(lib):
         _req(G == 1 and KD == kv_rank + rot_dim and v_cache.shape == (NB, 1, kv_rank, BS) and BS % 16 == 0,
              "latent cache: K [NB, 1, BS, kv_rank + rot_dim], V [NB, 1, kv_rank, BS], BS % 16 == 0")
         _check(lib.bcg_latent_kv_write(_p(y), y.stride(0), off, kv_rank, rot_dim, _p(w), eps, _p(positions), _p(slots),
-                                       _p(inv_freq), half, float(amp), _p(k_cache), _p(v_cache), T, BS, NB, _act(y), _stream()),
+                                       _p(inv_freq), half, float(amp), int(pairs), _p(k_cache), _p(v_cache), T, BS, NB, _act(y), _stream()),
                "latent_kv_write")
 
-    def rope_half_tail(src, src_off, dst, dst_off, positions, inv_freq, amp):
+    def rope_tail(src, src_off, dst, dst_off, positions, inv_freq, amp, pairs=False):
         _req(src.dim() == 3 and dst.dim() == 3 and src.is_contiguous() and dst.is_contiguous() and src.dtype == dst.dtype
-             and src.shape[:2] == dst.shape[:2], "rope_half_tail: src [T, H, Ds], dst [T, H, Dd] contiguous")
+             and src.shape[:2] == dst.shape[:2], "rope_tail: src [T, H, Ds], dst [T, H, Dd] contiguous")
         T, H, Ds = src.shape
         Dd = dst.shape[2]
         _req(0 <= src_off <= Ds and Ds - src_off == Dd - dst_off, "tails of equal width")
@@ -116,8 +149,8 @@ def seqlatent_ops(lib):
         half = inv_freq.numel()
         _f32(inv_freq, half, "inv_freq")
         _req(2 * half <= Ds - src_off, "rotated width <= tail")
-        _check(lib.bcg_rope_half_tail(_p(src), Ds, src_off, _p(dst), Dd, dst_off, _p(positions), _p(inv_freq), half, float(amp),
-                                      T, H, _act(src), _stream()), "rope_half_tail")
+        _check(lib.bcg_rope_tail(_p(src), Ds, src_off, _p(dst), Dd, dst_off, _p(positions), _p(inv_freq), half, float(amp),
+                                 int(pairs), T, H, _act(src), _stream()), "rope_tail")
         return dst
 
     def head_linear(x3, w, out3=None):
@@ -143,11 +176,11 @@ def seqlatent_ops(lib):
                                 group, _act(x), _stream()), "gate_mul")
         return out
 
-    def gated_act(both, kind="silu"):
-        _req(both.dim() == 2 and both.is_contiguous() and both.shape[1] % 2 == 0 and kind in ("silu", "gelu_tanh"),
-             "gated_act: [rows, 2 n] contiguous, silu or gelu_tanh")
+    def gated_act(both, kind="silu", limit=0.0):
+        _req(both.dim() == 2 and both.is_contiguous() and both.shape[1] % 2 == 0 and kind in ("silu", "gelu_tanh", "clamped_glu")
+             and (kind != "clamped_glu" or limit > 0), "gated_act: [rows, 2 n] contiguous, silu, gelu_tanh or clamped_glu (limit > 0)")
         out = torch.empty(both.shape[0], both.shape[1] // 2, dtype=both.dtype, device=both.device)
-        _check(lib.bcg_gated_act(_p(both), _p(out), both.shape[0], both.shape[1] // 2, ACT_CODES[kind], _act(both),
+        _check(lib.bcg_gated_act(_p(both), _p(out), both.shape[0], both.shape[1] // 2, ACT_CODES[kind], float(limit), _act(both),
                                  _stream()), "gated_act")
         return out
 
@@ -197,6 +230,6 @@ def seqlatent_ops(lib):
         return out
 
     return dict(embed_scale_dyt=embed_scale_dyt, residual_post_norm=residual_post_norm, rmsnorm_cols=rmsnorm_cols,
-                latent_kv_write=latent_kv_write, rope_half_tail=rope_half_tail, head_linear=head_linear, gate_mul=gate_mul,
+                latent_kv_write=latent_kv_write, rope_tail=rope_tail, head_linear=head_linear, gate_mul=gate_mul,
                 ssm_prepare=ssm_prepare, gated_group_norm=gated_group_norm, moe_table_route=moe_table_route,
                 gelu_gather_mul=gelu_gather_mul, gated_act=gated_act)

@@ -37,21 +37,23 @@ def _act(t):
     return int(t.dtype == torch.float32)
 
 
-ACT_CODES = {"gelu_tanh": 0, "relu2": 1, "silu": 2}
+ACT_CODES = {"gelu_tanh": 0, "relu2": 1, "silu": 2, "clamped_glu": 3}
+EXPERT_ACTS = {"silu_gated": "silu", "clamped_glu": "clamped_glu"}   # gated experts -> activation of their hidden values
 
 
 def seqmix_ops(lib, linear):
     split_keys = lib.bcg_multimap_split_keys()
     tile_rows = lib.bcg_moe_tile_rows()
 
-    def embed_scale_rmsnorm(tokens, table, scale, w, eps, w_offset, out_dtype):
+    def embed_scale_rmsnorm(tokens, table, scale, w, eps, w_offset, out_dtype, add=None):
         _req(tokens.dtype == torch.int32 and tokens.is_contiguous() and tokens.dim() == 1, "tokens int32 [T]")
         _req(table.dim() == 2 and table.is_contiguous() and table.dtype == out_dtype, "table [V, W] in the activation dtype")
         T, W = tokens.numel(), table.shape[1]
         _req(w.dtype == torch.float32 and w.shape == (W,) and w.is_contiguous(), "norm weight fp32 [W]")
+        _req(add is None or (add.dtype == torch.float32 and add.shape == (W,) and add.is_contiguous()), "added vector fp32 [W]")
         resid = torch.empty(T, W, dtype=torch.float32, device=table.device)
         out = torch.empty(T, W, dtype=out_dtype, device=table.device)
-        _check(lib.bcg_embed_scale_rmsnorm(_p(tokens), _p(table), scale, _p(w), eps, w_offset, _p(resid), _p(out), T, W,
+        _check(lib.bcg_embed_scale_rmsnorm(_p(tokens), _p(table), scale, _p(add), _p(w), eps, w_offset, _p(resid), _p(out), T, W,
                                            table.shape[0], _act(table), _stream()), "embed_scale_rmsnorm")
         return out, resid
 
@@ -154,13 +156,14 @@ def seqmix_ops(lib, linear):
         return 64  # four waves x 16 rows
 
     def multimap_attention(q, k_cache, v_cache, meta, scale, maps, lam, head_eps, out_scale, vdim, window=0, sink=None,
-                           chunk=0, softcap=0.0, slopes=None):
+                           chunk=0, softcap=0.0, slopes=None, keep=0):
         """Prefill tiles (``meta.tiles``) on the MFMA kernel, one-token rows (``meta.single``, or
         every row of a decode step) on the split-KV kernel.  ``window`` / ``chunk`` / ``sink``
         (one-map heads): sliding window in keys, or a chunk mask (a query sees the keys of its own
         ``chunk``-aligned block of positions only); fp32 [H] sink logits of the softmax denominator.
         ``softcap`` / ``slopes`` (one-map heads): scaled scores capped by tanh, then fp32 [H] slopes
-        times the distance to the key taken off."""
+        times the distance to the key taken off.  ``keep`` (with a window): the sequence's first ``keep``
+        keys stay visible."""
         T, H, qd = q.shape
         _req(q.is_contiguous() and qd % maps == 0, "q [T, H, maps dim] contiguous")
         dim = qd // maps
@@ -185,13 +188,15 @@ def seqmix_ops(lib, linear):
         _req(softcap >= 0 and (maps == 1 or (softcap == 0 and slopes is None)), "softcap / slopes: one-map heads")
         if slopes is not None:
             _req(slopes.dtype == torch.float32 and slopes.numel() == H and slopes.is_contiguous(), "slopes fp32 [H]")
+        keep = int(keep or 0) if window else 0   # (without a window nothing is hidden but the future)
+        _req(keep >= 0 and (keep == 0 or (softcap == 0 and slopes is None)), "kept first keys: without softcap / slopes")
         common = (H, G, maps, dim, vdim, BS, NB, scale, lam, head_eps, out_scale, tile_rows, f32, window, chunk, _p(sink), softcap,
-                  _p(slopes), _stream())
+                  _p(slopes), keep, _stream())
 
         def decode(work, n_items):
             n_splits = max(1, (bt.shape[1] * BS + split_keys - 1) // split_keys)
             if window or chunk:  # splits are counted from the window's (chunk's) first: it touches this many at most
-                n_splits = min(n_splits, (max(window, chunk) + split_keys - 1) // split_keys + 1)
+                n_splits = min(n_splits, (keep + split_keys - 1) // split_keys + (max(window, chunk) + split_keys - 1) // split_keys + 1)
             ws = torch.empty(n_items * H * n_splits * (2 * maps + maps * vdim), dtype=torch.float32, device=q.device)
             _check(lib.bcg_multimap_attention(1, _p(q), _p(k_cache), _p(v_cache), _p(bt), bt.shape[1], None, _p(lens),
                                               _p(work), n_items, _p(out), _p(ws), n_splits, *common), "multimap decode")
@@ -244,20 +249,21 @@ def seqmix_ops(lib, linear):
         return idx, wts
 
     def moe_pair_rows(gate, up):
-        """The [2 ff, W] weight of one gated expert as `moe_experts` (kind "silu_gated") reads it:
+        """The [2 ff, W] weight of one gated expert as `moe_experts` (kinds "silu_gated", "clamped_glu") reads it:
         gate and up rows in alternating groups of 16 when ff is a multiple of 16 (the product's
-        epilogue then forms silu(gate) * up), else [gate; up]."""
+        epilogue then forms the hidden values), else [gate; up]."""
         ff, W = gate.shape
         if ff % 16:
             return torch.cat([gate, up])
         return torch.stack([gate.reshape(ff // 16, 16, W), up.reshape(ff // 16, 16, W)], 1).reshape(2 * ff, W)
 
-    def moe_experts(h, up, down, idx, weights, kind="relu2"):
+    def moe_experts(h, up, down, idx, weights, kind="relu2", limit=0.0):
         T, W = h.shape
         E, n_up, _ = up.shape
         top = idx.shape[1]
-        _req(kind in ("relu2", "silu_gated"), "moe_experts: relu2 or silu-gated experts")
-        gated = kind == "silu_gated"
+        _req(kind == "relu2" or kind in EXPERT_ACTS, "moe_experts: relu2, silu-gated or clamped gated experts")
+        _req(kind != "clamped_glu" or limit > 0, "clamped experts: a positive limit")
+        gated = kind in EXPERT_ACTS
         _req(not gated or n_up % 2 == 0, "gated experts: [gate; up] rows")
         ff = n_up // 2 if gated else n_up
         _req(h.is_contiguous() and up.shape == (E, n_up, W) and down.shape == (E, W, ff) and up.is_contiguous()
@@ -271,23 +277,24 @@ def seqmix_ops(lib, linear):
         sorted_ = torch.empty(cap, dtype=torch.int32, device=dev)
         tile_e = torch.empty(n_tiles, dtype=torch.int32, device=dev)
         _check(lib.bcg_moe_align(_p(idx), n_slots, E, _p(sorted_), cap, _p(tile_e), n_tiles, _stream()), "moe_align")
-        if gated and ff % 16 == 0:   # rows paired by `moe_pair_rows`: silu(gate) * up in the product's epilogue
+        code = ACT_CODES[EXPERT_ACTS[kind]] if gated else 1
+        if gated and ff % 16 == 0:   # rows paired by `moe_pair_rows`: the hidden values in the product's epilogue
             hidden = torch.empty(cap, ff, dtype=h.dtype, device=dev)
-            _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(hidden), ff, _p(sorted_), _p(tile_e), n_tiles, n_up, W, top, 1, 0, 2,
-                                    f32, _stream()), "moe gate / up")
-        elif gated:   # the stacked projection, then silu(gate) * up over its halves
+            _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(hidden), ff, _p(sorted_), _p(tile_e), n_tiles, n_up, W, top, 1, 0, code,
+                                    limit, f32, _stream()), "moe gate / up")
+        elif gated:   # the stacked projection, then the hidden values from its halves
             both = torch.empty(cap, n_up, dtype=h.dtype, device=dev)
             _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(both), n_up, _p(sorted_), _p(tile_e), n_tiles, n_up, W, top, 1, 0, 0,
-                                    f32, _stream()), "moe gate / up")
+                                    0.0, f32, _stream()), "moe gate / up")
             hidden = torch.empty(cap, ff, dtype=h.dtype, device=dev)
-            _check(lib.bcg_gated_act(_p(both), _p(hidden), cap, ff, ACT_CODES["silu"], f32, _stream()), "gated_act")
+            _check(lib.bcg_gated_act(_p(both), _p(hidden), cap, ff, code, limit, f32, _stream()), "gated_act")
         else:
             hidden = torch.empty(cap, ff, dtype=h.dtype, device=dev)
             _check(lib.bcg_moe_gemm(_p(h), W, _p(up), _p(hidden), ff, _p(sorted_), _p(tile_e), n_tiles, ff, W, top, 1, 0, 1,
-                                    f32, _stream()), "moe up")
+                                    0.0, f32, _stream()), "moe up")
         y = torch.empty(n_slots, W, dtype=h.dtype, device=dev)
         _check(lib.bcg_moe_gemm(_p(hidden), ff, _p(down), _p(y), W, _p(sorted_), _p(tile_e), n_tiles, W, ff, top, 0, 1, 0,
-                                f32, _stream()), "moe down")
+                                0.0, f32, _stream()), "moe down")
         out = torch.empty(T, W, dtype=torch.float32, device=dev)
         _check(lib.bcg_moe_combine(_p(y), _p(weights), _p(out), T, W, top, f32, _stream()), "moe_combine")
         return out

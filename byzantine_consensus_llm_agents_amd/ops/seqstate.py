@@ -101,7 +101,7 @@ def seqstate_ops(lib):
         return out
 
     def rope_pairs_kv_write(qkv, positions, slots, n_q, n_kv, dim, vdim, q_norm, k_norm, eps, inv_freq, v_inv_freq,
-                            k_cache, v_cache, v_is_k=False, q_temp=None):
+                            k_cache, v_cache, v_is_k=False, q_temp=None, amp=1.0):
         T = qkv.shape[0]
         qw, kw, vw = n_q * dim, n_kv * dim, n_kv * vdim
         _req(not v_is_k or vdim == dim, "values that are the keys: vdim = dim")
@@ -128,7 +128,7 @@ def seqstate_ops(lib):
              "KV cache: K [NB, G, BS, dim], V [NB, G, vdim, BS], BS % 16 == 0")
         q = torch.empty(T, n_q, dim, dtype=qkv.dtype, device=qkv.device)
         _check(lib.bcg_rope_pairs_kv_write(_p(qkv), qkv.stride(0), _p(positions), _p(slots), _p(q_norm), _p(k_norm), eps,
-                                           _p(inv_freq), half, _p(v_inv_freq), _p(q), _p(k_cache), _p(v_cache), T, n_q, n_kv, dim,
+                                           _p(inv_freq), half, float(amp), _p(v_inv_freq), _p(q), _p(k_cache), _p(v_cache), T, n_q, n_kv, dim,
                                            vdim, v_off, coef, every, BS, NB, _act(qkv), _stream()), "rope_pairs_kv_write")
         return q
 
@@ -173,8 +173,23 @@ def seqstate_ops(lib):
                "delta_prepare")
         return q, k, g, beta
 
+    def retention_prepare(y, off_q, off_k, heads, dim, k_scale, positions, inv_freq, amp=1.0):
+        T, n = y.shape[0], heads * dim
+        _req(y.dim() == 2 and y.stride(1) == 1 and min(off_q, off_k) >= 0 and y.shape[1] >= max(off_q, off_k) + n,
+             "retention_prepare: fused projection rows")
+        _i32(positions, T, "positions")
+        half = inv_freq.numel()
+        _f32(inv_freq, half, "inv_freq")
+        _req(2 * half <= dim and half <= 4096, "rotated width <= dim, <= 4096 pairs")
+        q, k = (torch.empty(T, heads, dim, dtype=torch.float32, device=y.device) for _ in range(2))
+        _check(lib.bcg_retention_prepare(_p(y), y.stride(0), off_q, off_k, heads, dim, _p(positions), _p(inv_freq), half, float(amp),
+                                         float(k_scale), _p(q), _p(k), T, _act(y), _stream()), "retention_prepare")
+        return q, k
+
     def gated_state_scan(q, k, g, v, beta, meta, state, delta, unit_last=False):
-        T, H, gd = g.shape
+        T, g_const = q.shape[0], g.dim() == 1   # [H]: the same decays for every token
+        H, gd = (g.numel(), 1) if g_const else g.shape[1:]
+        _req(g_const or g.shape[0] == T, "g [T, H, dim], [T, H, 1] or [H]")
         _req(state.dim() == 4 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == H,
              "state fp32 [rows, H, dim, vdim]")
         dim = state.shape[2]
@@ -194,7 +209,7 @@ def seqstate_ops(lib):
         out = torch.empty(T, H, vdim, dtype=torch.float32, device=g.device)
         _check(lib.bcg_gated_state_scan(_p(q), _p(k), _p(g), _p(v), v.stride(0), _p(beta), _p(meta.positions),
                                         _p(meta.q_start), _p(meta.state_rows), _p(state), state.shape[0], _p(out), B, H, Gq, dim,
-                                        vdim, gd, int(bool(delta)), int(bool(unit_last)), _act(v), _stream()), "gated_state_scan")
+                                        vdim, gd, int(g_const), int(bool(delta)), int(bool(unit_last)), _act(v), _stream()), "gated_state_scan")
         return out
 
     def head_norm_gate(o, w, eps, gate, out_dtype, gate_act="sigmoid", floor=None):
@@ -203,8 +218,9 @@ def seqstate_ops(lib):
         if floor is not None:   # o's last column is a normaliser
             vdim -= 1
             _req(vdim >= 1 and floor.dtype == torch.float32 and floor.shape == (T, H) and floor.is_contiguous(), "floor fp32 [T, H]")
-        _req(w.numel() in (vdim, H * vdim), "head norm weight [vdim] or [H vdim]")
-        _f32(w, w.numel(), "head norm weight")
+        if w is not None:
+            _req(w.numel() in (vdim, H * vdim), "head norm weight [vdim] or [H vdim]")
+            _f32(w, w.numel(), "head norm weight")
         stride = 0
         if gate is not None:
             _req(gate.dim() == 2 and gate.stride(1) == 1 and gate.shape == (T, H * vdim) and gate.dtype == out_dtype,
@@ -212,7 +228,7 @@ def seqstate_ops(lib):
             stride = gate.stride(0)
         out = torch.empty(T, H * vdim, dtype=out_dtype, device=o.device)
         _check(lib.bcg_head_norm_gate(_p(o), _p(w), eps, _p(gate), stride, _p(out), T, H, vdim,
-                                      {"sigmoid": 0, "silu": 1}[gate_act], _p(floor), vdim if w.numel() != vdim else 0,
+                                      {"sigmoid": 0, "silu": 1}[gate_act], _p(floor), vdim if w is not None and w.numel() != vdim else 0,
                                       int(out_dtype == torch.float32), _stream()),
                "head_norm_gate")
         return out
@@ -220,4 +236,4 @@ def seqstate_ops(lib):
     return dict(embed_hashed_bigram_norm=embed_hashed_bigram_norm, residual_mix_norm=residual_mix_norm,
                 rmsnorm_scalar=rmsnorm_scalar, short_conv=short_conv, rope_pairs_kv_write=rope_pairs_kv_write,
                 rotate_pairs=rotate_pairs, hgrn2_prepare=hgrn2_prepare, delta_prepare=delta_prepare,
-                gated_state_scan=gated_state_scan, head_norm_gate=head_norm_gate)
+                gated_state_scan=gated_state_scan, retention_prepare=retention_prepare, head_norm_gate=head_norm_gate)

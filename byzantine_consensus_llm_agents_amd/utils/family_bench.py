@@ -453,7 +453,7 @@ def latent_kernels(s, dev):
     out["cache_write"].update({"padadra_ms": round(t * 1e3, 4), "padadra_roof_frac": _roof(0, T * width * 2 * 2, t)})
     # ---- query assembly: tail rotary into the packed query (the per-head products are vendor GEMMs) ----
     qsrc, qdst = torch.randn(T, H, 128 + RD, device=dev, dtype=bf), torch.empty(T, H, KD, device=dev, dtype=bf)
-    t = _graph_time(lambda: ops.rope_half_tail(qsrc, 128, qdst, R, meta.positions, inv, 1.2), iters=50)
+    t = _graph_time(lambda: ops.rope_tail(qsrc, 128, qdst, R, meta.positions, inv, 1.2), iters=50)
     out["query_tail_rotary"] = {"mabivik_ms": round(t * 1e3, 4), "mabivik_roof_frac": _roof(0, T * H * RD * 2 * 2, t)}
     # ---- routed experts: gated (three matrices, activation in the epilogue) against relu^2 (two matrices) ----
     E, top, ff = 8, 2, s["ff"] // 4

@@ -29,9 +29,12 @@
 // i - j < window) or a chunk mask (position i sees j <= i of its own chunk, floor(i / chunk) ==
 // floor(j / chunk), chunks counted from position 0), and a per-head sink, a learned logit that takes part in the softmax denominator
 // only (no key, no value, not scaled).  The key loop starts at the window's (chunk's) first 16-key
-// tile; decode splits are counted from the window's (chunk's) first split.
+// tile; decode splits are counted from the window's (chunk's) first split.  A window may keep the
+// sequence's first `keep` keys (KEEP instances): every query sees them at their true positions.  The
+// key loop then walks the tiles of the kept keys, jumps to the window's first tile and goes on; decode
+// splits are those that hold kept keys, then the window's.
 //
-// Optional score shape (SC instances, one-map heads): the scaled score s becomes cap tanh(s / cap)
+// Optional score shape (SHAPED instances, one-map heads): the scaled score s becomes cap tanh(s / cap)
 // (cap > 0), then slope_h (i - j) is taken off (slopes non-null).  Both act on fp32 scores.
 #include <algorithm>
 
@@ -40,6 +43,7 @@
 namespace {
 
 constexpr int SPLIT_KEYS = 128;
+constexpr int PLAIN = 0, SHAPED = 1, KEEP = 2;   // loop forms: as is / capped or biased scores / kept first keys
 constexpr float MAX_FLOOR = -1.0e30f;   // running maxima start finite: a tile may be hidden as a whole
 constexpr float LOG2E = 1.4426950408889634f;
 
@@ -57,10 +61,11 @@ struct AttnArgs {
   float scale, lam, head_eps, out_scale;
   int vec_k, vec_v;         // rows of K / V^T are aligned for 4-element vector loads
   int window;               // > 0: keys below position - window + 1 are hidden
+  int keep;                 // > 0 (with a window): keys below `keep` stay visible (KEEP instances)
   int chunk;                // > 0: keys below position - position % chunk are hidden (chunks count from position 0)
   const float* sink;        // [H] or null
-  float softcap;            // > 0: scaled scores are capped, cap tanh(s / cap)   (SC instances)
-  const float* slopes;      // [H] or null: slope_h (i - j) is taken off the score (SC instances)
+  float softcap;            // > 0: scaled scores are capped, cap tanh(s / cap)   (SHAPED instances)
+  const float* slopes;      // [H] or null: slope_h (i - j) is taken off the score (SHAPED instances)
   int swz;                  // fragment-major slabs (see the top of the file)
 };
 
@@ -71,6 +76,18 @@ __device__ __forceinline__ int first_key(const AttnArgs& a, int pos) {
   return 0;
 }
 
+// Decode splits of a row whose window starts at key `lo`: split i covers the keys of the absolute split
+// `split_abs` -- first those that hold kept keys, then the window's.
+__device__ __forceinline__ int keep_splits(const AttnArgs& a) { return (a.keep + SPLIT_KEYS - 1) / SPLIT_KEYS; }
+__device__ __forceinline__ int split_abs_of(const AttnArgs& a, int lo, int split) {
+  const int nk = keep_splits(a);
+  return split < nk ? split : max(lo / SPLIT_KEYS, nk) + split - nk;
+}
+__device__ __forceinline__ int split_count(const AttnArgs& a, int lo, int ctx) {
+  const int nk = keep_splits(a), total = (ctx + SPLIT_KEYS - 1) / SPLIT_KEYS;
+  return total <= nk ? total : nk + total - max(lo / SPLIT_KEYS, nk);
+}
+
 // The key loop shared by both kernels: keys [k_begin, k_last] of one sequence for the 16 query
 // columns of a wave (column = a query row of one head, or a query head of one token).
 //   limit      per lane: the last key its column may see;  limit_min: the smallest over the wave
@@ -79,16 +96,18 @@ __device__ __forceinline__ int first_key(const AttnArgs& a, int pos) {
 //   PF         this iteration's V^T fragments are loaded before its QK^T products and the next
 //              iteration's K fragments right after them (loads fly under the MFMAs and the softmax)
 //   FULL       whole, aligned fragments only (no branch around any load)
-//   SC         scores are capped / biased: pos = the position of the lane's column, slope = its head's
-//              slope times log2 e
+//   MODE       SHAPED: scores are capped / biased: pos = the position of the lane's column, slope = its head's
+//              slope times log2 e.  KEEP: keys below `keep` stay visible; once they are passed the loop
+//              jumps to the tile at k_win (a multiple of 16)
 // Everything that does not depend on the lane stays scalar: the page lookup and the slab base go
 // to SGPRs, a lane adds a 32-bit offset that is fixed for the whole loop.  Scores are kept in the
 // log2 domain (scale * log2 e folded into one multiply, v_exp_f32 directly).
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int EXACT, int NM, bool SC>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int EXACT, int NM, int MODE>
 __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const typename Elem<T>::frag (&qf)[NM][KC],
                                              int limit, int limit_min, int lo, int lo_max, int k_begin, int k_last,
                                              const int* __restrict__ table, f32x4 (&acc)[NM][VT], float (&mx)[NM],
-                                             float (&den)[NM], int pos = 0, float slope = 0.f) {
+                                             float (&den)[NM], int pos = 0, float slope = 0.f, int keep = 0,
+                                             int k_win = 0) {
   typedef typename Elem<T>::frag F;
   // EXACT (1 or 2 = the number of maps): dim = 16 KC, vdim = 16 VT, 16-token pages, fragment-major slabs -- every guard
   // below is a compile-time constant, fragment offsets are immediates, the loop body is straight-line
@@ -106,7 +125,7 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
   const bool vec_k = a.vec_k && (a.dim & 3) == 0;
   const float sc = a.scale * 1.4426950408889634f;
   // capped scores: cap tanh(s / cap) = cap - 2 cap / (exp(2 s / cap) + 1), in the log2 domain
-  const float cap = SC ? a_.softcap : 0.f;
+  const float cap = MODE == SHAPED ? a_.softcap : 0.f;
   const float cap2 = cap * LOG2E, arg2 = cap > 0.f ? 2.0f * LOG2E * a.scale / cap : 0.f;
   auto shape_score = [&](float dot, int key, bool capped) {
     float v = dot * sc;
@@ -135,6 +154,16 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
     c.o += 16;
     if (c.o >= a.BS) { c.o = 0; ++c.p; }
   };
+  auto place = [&](Cursor& c, int key) {
+    c.p = key / a.BS;
+    c.o = key - c.p * a.BS;
+  };
+  // first key of the iteration behind the one at `key0`; KEEP: past the kept keys, on to the window
+  auto next_key = [&](int key0) {
+    const int n = key0 + 16 * KT;
+    if constexpr (MODE == KEEP) return (n >= keep && n < k_win) ? k_win : n;
+    else return n;
+  };
   auto slab_base = [&](const Cursor& c) {
     int page = table[min(c.p, a.max_blocks - 1)];
     page = (page < 0 || page >= a.num_blocks) ? 0 : page;
@@ -155,17 +184,23 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
   };
 
   Cursor k_cur, v_cur;
-  k_cur.p = k_begin / a.BS;
-  k_cur.o = k_begin - k_cur.p * a.BS;
+  place(k_cur, k_begin);
   v_cur = k_cur;
   F kf[KT][NM][KC];
   if (PF) load_k(k_cur, kf);
-  for (int key0 = k_begin; key0 <= k_last; key0 += 16 * KT) {
+  for (int key0 = k_begin, key_next; key0 <= k_last; key0 = key_next) {
+    key_next = next_key(key0);
     const T* vps[KT];
 #pragma unroll
     for (int u = 0; u < KT; ++u) {
       vps[u] = vc_base + slab_base(v_cur) * v_slab + v_cur.o * v_mul;
       step(v_cur);
+    }
+    if constexpr (MODE == KEEP) {
+      if (key_next != key0 + 16 * KT) {   // (wave-uniform) the jump
+        place(v_cur, key_next);
+        if (PF) place(k_cur, key_next);
+      }
     }
     F vf[PF ? KT : 1][PF ? VT : 1];
     auto load_v = [&](int u, int t) {
@@ -178,6 +213,9 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
         for (int t = 0; t < VT; ++t) vf[u][t] = load_v(u, t);
     } else {
       load_k(k_cur, kf);
+      if constexpr (MODE == KEEP) {
+        if (key_next != key0 + 16 * KT) place(k_cur, key_next);
+      }
     }
     // ---- S^T = K Q^T ----
     f32x4 s[KT][NM];
@@ -194,12 +232,12 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
       }
     // the K fragments are spent: the next iteration's go into the same registers, under the
     // softmax and the second product
-    if (PF && key0 + 16 * KT <= k_last) load_k(k_cur, kf);
+    if (PF && key_next <= k_last) load_k(k_cur, kf);
     // ---- online softmax per query column; lane holds keys key0 + 16 u + 4 grp + i ----
     const bool masked = key0 + 16 * KT - 1 > limit_min || key0 < lo_max;   // (wave-uniform) some key of the iteration is hidden
     // (opaque per iteration: one loop body, not one per combination of uniform conditions)
     float cap_now = cap;
-    if constexpr (SC) asm volatile("" : "+v"(cap_now));
+    if constexpr (MODE == SHAPED) asm volatile("" : "+v"(cap_now));
     const bool capped = cap_now > 0.f;
     F pf[KT][NM];
 #pragma unroll
@@ -214,9 +252,10 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
       for (int u = 0; u < KT; ++u)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          if constexpr (SC) v[u][i] = shape_score(s[u][m][i], key0 + 16 * u + 4 * grp + i, capped);
+          const int key = key0 + 16 * u + 4 * grp + i;
+          if constexpr (MODE == SHAPED) v[u][i] = shape_score(s[u][m][i], key, capped);
           else v[u][i] = s[u][m][i] * sc;
-          if (masked && (key0 + 16 * u + 4 * grp + i > limit || key0 + 16 * u + 4 * grp + i < lo)) v[u][i] = -INFINITY;
+          if (masked && (key > limit || (key < lo && !(MODE == KEEP && key < keep)))) v[u][i] = -INFINITY;
           bm = fmaxf(bm, v[u][i]);
         }
       bm = fmaxf(bm, __shfl_xor(bm, 16, WAVE));
@@ -260,7 +299,7 @@ __device__ __forceinline__ void attend_range(const AttnArgs& a_, int g, const ty
   }
 }
 
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, bool SC = false>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, int MODE = PLAIN>
 __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
   typedef typename Elem<T>::frag F;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -302,10 +341,11 @@ __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
     den[0] = 1.0f;
   }
   const int lo = first_key(a, pos), lo_max = first_key(a, pos_max);   // (both masks: the first key grows with the position)
-  const int k_begin = first_key(a, pos_min) & ~15;
-  const float slope = SC && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
-  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, SC>(a, g, qf, pos, pos_min, lo, lo_max, k_begin, pos_max,
-                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, pos, slope);
+  const int k_win = first_key(a, pos_min) & ~15, k_begin = MODE == KEEP ? 0 : k_win;
+  const float slope = MODE == SHAPED && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
+  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, MODE>(a, g, qf, pos, pos_min, lo, lo_max, k_begin, pos_max,
+                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, pos, slope,
+                                        a.keep, k_win);
   // ---- combine the maps, unit norm over the head's value features, store ----
   const float i0 = 1.0f / den[0];
   float i1 = 0.f;
@@ -347,7 +387,7 @@ __global__ __launch_bounds__(256, OCC) void prefill_kernel(AttnArgs a) {
 // head g (H / G) + 16 cg + c of the same token, so K and V^T are read once per KV head.  One wave
 // per (item, KV head x column group, SPLIT_KEYS-key split); partials as the merge kernel reads them
 // (running maxima in the log2 domain of `attend_range`).
-template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, bool SC = false>
+template <typename T, int KC, int VT, int KT, bool PF, bool FULL, int OCC, int EXACT = 0, int NM = 2, int MODE = PLAIN>
 __global__ __launch_bounds__(64, OCC) void decode_mfma_kernel(AttnArgs a) {
   typedef typename Elem<T>::frag F;
   const int lane = threadIdx.x, col = lane & 15, grp = lane >> 4;
@@ -357,9 +397,14 @@ __global__ __launch_bounds__(64, OCC) void decode_mfma_kernel(AttnArgs a) {
   const int row = a.work ? a.work[2 * item] : item, seq = a.work ? a.work[2 * item + 1] : item;
   const int ctx = a.seq_lens[seq];
   const int lo = first_key(a, ctx - 1);                             // first visible key
-  const int split_abs = lo / SPLIT_KEYS + split;                    // splits count from the window's first
-  const int k_end = min(ctx, (split_abs + 1) * SPLIT_KEYS);
-  const int k_begin = max(split_abs * SPLIT_KEYS, lo & ~15);
+  const int split_abs = MODE == KEEP ? split_abs_of(a, lo, split) : lo / SPLIT_KEYS + split;   // splits count from the window's first
+  int k_end = min(ctx, (split_abs + 1) * SPLIT_KEYS);
+  const int k_win = max(split_abs * SPLIT_KEYS, lo & ~15);
+  int k_begin = k_win;
+  if constexpr (MODE == KEEP) {
+    if (split_abs * SPLIT_KEYS < a.keep) k_begin = split_abs * SPLIT_KEYS;   // the split holds kept keys ...
+    if (lo >= k_end) k_end = min(k_end, a.keep);                             // ... and none of the window's
+  }
   if (k_begin >= k_end) return;
   const bool col_ok = 16 * cg + col < per;
   const int h = g * per + min(16 * cg + col, per - 1);
@@ -386,9 +431,10 @@ __global__ __launch_bounds__(64, OCC) void decode_mfma_kernel(AttnArgs a) {
     mx[m] = MAX_FLOOR;
     den[m] = 0.f;
   }
-  const float slope = SC && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
-  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, SC>(a, g, qf, k_end - 1, k_end - 1, lo, lo, k_begin, k_end - 1,
-                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, ctx - 1, slope);
+  const float slope = MODE == SHAPED && a.slopes != nullptr ? a.slopes[h] * LOG2E : 0.f;
+  attend_range<T, KC, VT, KT, PF, FULL, EXACT, NM, MODE>(a, g, qf, k_end - 1, k_end - 1, lo, lo, k_begin, k_end - 1,
+                                        a.block_tables + static_cast<size_t>(seq) * a.max_blocks, acc, mx, den, ctx - 1, slope,
+                                        a.keep, k_win);
   if (!col_ok) return;
   float* w = a.ws + ((static_cast<size_t>(item) * a.H + h) * a.n_splits + split) * (2 * a.maps + a.maps * a.vdim);
 #pragma unroll
@@ -416,8 +462,7 @@ __global__ __launch_bounds__(64) void decode_merge_kernel(AttnArgs a) {
   const int lane = threadIdx.x, h = blockIdx.x, item = blockIdx.y;
   const int row = a.work ? a.work[2 * item] : item, seq = a.work ? a.work[2 * item + 1] : item;
   const int ctx = a.seq_lens[seq];
-  const int s_first = first_key(a, ctx - 1) / SPLIT_KEYS;
-  const int n = min(a.n_splits, (ctx + SPLIT_KEYS - 1) / SPLIT_KEYS - s_first);
+  const int n = min(a.n_splits, split_count(a, first_key(a, ctx - 1), ctx));
   const float sink = a.sink != nullptr ? a.sink[h] * LOG2E : MAX_FLOOR;
   const int stride = 2 * a.maps + a.maps * a.vdim;
   const float* w = a.ws + (static_cast<size_t>(item) * a.H + h) * a.n_splits * stride;
@@ -459,41 +504,42 @@ __global__ __launch_bounds__(64) void decode_merge_kernel(AttnArgs a) {
 // Exact one-map instances (bf16): X(KC, VT, keys tiles per iteration, workgroups per CU).
 #define BCG_EXACT1_PLAIN(X) X(8, 8, 2, 2) X(4, 4, 2, 2) X(4, 8, 2, 2) X(2, 2, 2, 2) X(6, 6, 2, 2) X(6, 4, 2, 2) X(12, 8, 2, 2) \
                             X(12, 12, 2, 1) X(16, 16, 2, 1) X(32, 32, 1, 1)
+#define BCG_EXACT1_KEEP(X) X(8, 8, 2, 2) X(4, 4, 2, 2) X(4, 8, 2, 2) X(2, 2, 2, 2) X(6, 6, 2, 2) X(12, 12, 2, 1) X(16, 16, 2, 1)
 #define BCG_EXACT1_SHAPED(X) X(8, 8, 2, 2) X(4, 4, 2, 2) X(2, 2, 2, 2) X(3, 3, 2, 2) X(6, 6, 2, 2) X(12, 12, 2, 1) X(16, 16, 2, 1)
 
-// Heads whose scores are capped or biased (one map).
-template <typename T>
-int launch_prefill_shaped(const AttnArgs& a, int n_tiles, bool full, hipStream_t s) {
+// Heads whose scores are capped or biased, or whose window keeps first keys (one map).
+template <typename T, int MODE>
+int launch_prefill_mode(const AttnArgs& a, int n_tiles, bool full, hipStream_t s) {
   dim3 grid(n_tiles, a.H);
   if constexpr (sizeof(T) == 2) if (full && a.swz && a.BS == 16) {
 #define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
-    prefill_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, true><<<grid, 256, 0, s>>>(a);      \
+    prefill_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, MODE><<<grid, 256, 0, s>>>(a);      \
     return BCG_CHECK_LAUNCH();                                                                   \
   }
-    BCG_EXACT1_SHAPED(BCG_X)
+    if constexpr (MODE == SHAPED) { BCG_EXACT1_SHAPED(BCG_X) } else { BCG_EXACT1_KEEP(BCG_X) }
 #undef BCG_X
   }
-  if (a.dim <= 64 && a.vdim <= 128) prefill_kernel<T, 4, 8, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
-  else if (a.dim <= 256 && a.vdim <= 256) prefill_kernel<T, 16, 16, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
-  else prefill_kernel<T, 32, 32, 1, false, false, 1, 0, 1, true><<<grid, 256, 0, s>>>(a);
+  if (a.dim <= 64 && a.vdim <= 128) prefill_kernel<T, 4, 8, 1, false, false, 1, 0, 1, MODE><<<grid, 256, 0, s>>>(a);
+  else if (a.dim <= 256 && a.vdim <= 256) prefill_kernel<T, 16, 16, 1, false, false, 1, 0, 1, MODE><<<grid, 256, 0, s>>>(a);
+  else prefill_kernel<T, 32, 32, 1, false, false, 1, 0, 1, MODE><<<grid, 256, 0, s>>>(a);
   return BCG_CHECK_LAUNCH();
 }
 
-template <typename T>
-void launch_decode_shaped(const AttnArgs& a, dim3 grid, bool full, hipStream_t s) {
+template <typename T, int MODE>
+void launch_decode_mode(const AttnArgs& a, dim3 grid, bool full, hipStream_t s) {
   if constexpr (sizeof(T) == 2) if (full && a.swz && a.BS == 16) {
 #define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
-    decode_mfma_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, true><<<grid, 64, 0, s>>>(a);   \
+    decode_mfma_kernel<T, KC_, VT_, KT_, true, true, OCC_, 1, 1, MODE><<<grid, 64, 0, s>>>(a);   \
     return;                                                                                      \
   }
-    BCG_EXACT1_SHAPED(BCG_X)
+    if constexpr (MODE == SHAPED) { BCG_EXACT1_SHAPED(BCG_X) } else { BCG_EXACT1_KEEP(BCG_X) }
 #undef BCG_X
   }
-  if (a.dim <= 64 && a.vdim <= 128) decode_mfma_kernel<T, 4, 8, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
-  else if (a.dim <= 256 && a.vdim <= 256) decode_mfma_kernel<T, 16, 16, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
-  else decode_mfma_kernel<T, 32, 32, 1, false, false, 1, 0, 1, true><<<grid, 64, 0, s>>>(a);
+  if (a.dim <= 64 && a.vdim <= 128) decode_mfma_kernel<T, 4, 8, 1, false, false, 1, 0, 1, MODE><<<grid, 64, 0, s>>>(a);
+  else if (a.dim <= 256 && a.vdim <= 256) decode_mfma_kernel<T, 16, 16, 1, false, false, 1, 0, 1, MODE><<<grid, 64, 0, s>>>(a);
+  else decode_mfma_kernel<T, 32, 32, 1, false, false, 1, 0, 1, MODE><<<grid, 64, 0, s>>>(a);
 }
 
 template <typename T>
@@ -502,7 +548,8 @@ int launch_prefill(const AttnArgs& a, int n_tiles, int tile_rows, hipStream_t s)
   const bool small = a.dim <= 64 && a.vdim <= 128;
   const bool full = a.dim % 16 == 0 && a.vdim % 16 == 0 && a.vec_k && a.vec_v;   // whole, aligned fragments only
   if (tile_rows != 64) return -2;
-  if (a.softcap > 0.f || a.slopes != nullptr) return launch_prefill_shaped<T>(a, n_tiles, full, s);
+  if (a.softcap > 0.f || a.slopes != nullptr) return launch_prefill_mode<T, SHAPED>(a, n_tiles, full, s);
+  if (a.keep > 0) return launch_prefill_mode<T, KEEP>(a, n_tiles, full, s);
   if constexpr (sizeof(T) == 2) if (full && a.maps == 1 && a.swz && a.BS == 16) {   // one-map heads, exact shapes
 #define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                                 \
@@ -545,8 +592,10 @@ int launch_decode(const AttnArgs& a, int n_items, hipStream_t s) {
   const int per = a.H / a.G;
   dim3 grid(a.G * ((per + 15) / 16), a.n_splits, n_items);
   const bool full = a.dim % 16 == 0 && a.vdim % 16 == 0 && a.vec_k && a.vec_v;
-  bool done = a.softcap > 0.f || a.slopes != nullptr;
-  if (done) launch_decode_shaped<T>(a, grid, full, s);
+  const bool shaped = a.softcap > 0.f || a.slopes != nullptr;
+  bool done = shaped || a.keep > 0;
+  if (shaped) launch_decode_mode<T, SHAPED>(a, grid, full, s);
+  else if (done) launch_decode_mode<T, KEEP>(a, grid, full, s);
   if constexpr (sizeof(T) == 2) if (!done && full && a.maps == 1 && a.swz && a.BS == 16) {   // one-map heads, exact shapes
 #define BCG_X(KC_, VT_, KT_, OCC_)                                                               \
   if (!done && a.dim == 16 * KC_ && a.vdim == 16 * VT_) {                                        \
@@ -602,8 +651,9 @@ BCG_API int bcg_multimap_attention(int mode, const void* q, const void* k_cache,
                                    const void* work, int n_work, void* out, void* ws, int n_splits, int H, int G, int maps,
                                    int dim, int vdim, int BS, int num_blocks, float scale, float lam, float head_eps,
                                    float out_scale, int tile_rows, int is_f32, int window, int chunk, const void* sink,
-                                   float softcap, const void* slopes, void* stream) {
+                                   float softcap, const void* slopes, int keep, void* stream) {
   if (n_work <= 0) return 0;
+  if (keep < 0 || (keep > 0 && (window <= 0 || softcap != 0.f || slopes != nullptr))) return -2;
   if ((window > 0 || chunk > 0 || sink != nullptr || softcap != 0.f || slopes != nullptr) && maps != 1) return -2;
   if (window > 0 && chunk > 0) return -2;
   if (maps < 1 || maps > 2 || dim > (maps == 1 ? 512 : 128) || vdim > (maps == 1 ? 512 : 256) || BS % 16 || H % G || n_work > 65535 * 16) return -2;
@@ -618,7 +668,7 @@ BCG_API int bcg_multimap_attention(int mode, const void* q, const void* k_cache,
   a.vec_k = ((maps * dim) % 4 == 0) ? 1 : 0;
   a.vec_v = 1;  // BS % 16 == 0: every 4-key group of a V^T row is aligned
   a.swz = a.vec_k;
-  a.window = window; a.chunk = chunk; a.sink = static_cast<const float*>(sink);
+  a.window = window; a.keep = keep; a.chunk = chunk; a.sink = static_cast<const float*>(sink);
   a.softcap = softcap; a.slopes = static_cast<const float*>(slopes);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (mode == 0) return is_f32 ? launch_prefill<float>(a, n_work, tile_rows, s) : launch_prefill<bf16_t>(a, n_work, tile_rows, s);

@@ -67,6 +67,12 @@ __device__ __forceinline__ typename Elem<T>::frag load_frag_t(const T* p, int n_
   else return load_frag<T>(p, n_valid, vec);
 }
 
+// Clamped gated unit: g = min(gate, limit), u = up clamped to +-limit, g sigmoid(1.702 g) (u + 1).
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+
 template <typename T>
 __device__ __forceinline__ typename Elem<T>::frag zero_frag() {
   typename Elem<T>::frag r;

@@ -5,8 +5,8 @@
 //   dynamic-tanh norm (alpha, w, b):  tanh(alpha x) w + b   -- elementwise, no row statistic
 //   latent cache of a token:          K row = [rms(c) w | turned shared key part],  V^T column = rms(c) w
 //                                     in the slab layout of seqmix_attention.hip with ONE KV head
-//   rotary:                           feature i of the turned part pairs with i + half; cos and sin
-//                                     both carry an amplitude (frequency-scaled rotary)
+//   rotary:                           feature i of the turned part pairs with i + half, or 2i with 2i + 1
+//                                     (pairs); cos and sin both carry an amplitude (frequency-scaled rotary)
 //
 // T is the activation type (bf16 bits or float); the stream, the norms, angles, decays and step
 // sizes are fp32.
@@ -132,26 +132,44 @@ __global__ __launch_bounds__(NT) void residual_post_norm_kernel(float* __restric
   }
 }
 
-// ---------------------------------------------------------------- x += layer_norm(y); out = x rounded | layer_norm(x)
+// ---------------------------------------------------------------- x += norm(y) + entry; out = x rounded | norm(x)
 // One workgroup per row, which stays in registers: NV chunks of V columns per thread (NV * V * NT >= W;
-// V = 4: 8- / 16-byte accesses).  pre_kind 0: nothing; 1: x rounded to T; 2: the layer norm (qw, qb) of
-// the new x.  Mean first, then the squared deviations.
-template <typename T, typename Y, int V, int NV>
-__global__ __launch_bounds__(NT) void residual_layer_norm_kernel(float* __restrict__ resid, const Y* __restrict__ y,
-                                                                 const float* __restrict__ w, const float* __restrict__ b, float eps,
-                                                                 int pre_kind, const float* __restrict__ qw,
-                                                                 const float* __restrict__ qb, float pre_eps, T* __restrict__ out,
-                                                                 int W) {
+// V = 4: 8- / 16-byte accesses).  pre_kind 0: nothing; 1: x rounded to T; 2: the norm (qw, qb) of
+// the new x.  LN: both norms are layer norms with weight and bias (mean first, then the squared
+// deviations); else RMS norms with a weight.  Without LN, y may be null (no sublayer output) and the
+// stream may take an entry behind the norm: the vector `add`, and the row's token row of `table`.
+struct StreamEntry {
+  const float* add;     // [W] or null: no entry
+  const int* tokens;    // [rows]
+  const void* table;    // [vocab, W] of the activation type, or null: only the vector
+  int vocab;
+};
+
+template <typename T, typename Y, int V, int NV, bool LN>
+__global__ __launch_bounds__(NT) void residual_row_norm_kernel(float* __restrict__ resid, const Y* __restrict__ y,
+                                                               const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                               int pre_kind, const float* __restrict__ qw,
+                                                               const float* __restrict__ qb, float pre_eps, T* __restrict__ out,
+                                                               int W, StreamEntry entry) {
   __shared__ float red[NT / 64];
   const size_t base = static_cast<size_t>(blockIdx.x) * W;
+  const bool has_y = LN || y != nullptr;
+  const T* trow = nullptr;
+  if constexpr (!LN) {
+    if (entry.add != nullptr && entry.table != nullptr)
+      trow = static_cast<const T*>(entry.table) + static_cast<size_t>(min(max(entry.tokens[blockIdx.x], 0), entry.vocab - 1)) * W;
+  }
   float v[NV][V];
   auto stats = [&](float e, float& mean, float& r) {
-    float s = 0.f;
+    mean = 0.f;
+    if constexpr (LN) {
+      float s = 0.f;
 #pragma unroll
-    for (int k = 0; k < NV; ++k)
+      for (int k = 0; k < NV; ++k)
 #pragma unroll
-      for (int j = 0; j < V; ++j) s += v[k][j];   // (columns past the row hold zeros)
-    mean = block_sum(s, red) / W;
+        for (int j = 0; j < V; ++j) s += v[k][j];   // (columns past the row hold zeros)
+      mean = block_sum(s, red) / W;
+    }
     float sq = 0.f;
 #pragma unroll
     for (int k = 0; k < NV; ++k)
@@ -169,7 +187,7 @@ __global__ __launch_bounds__(NT) void residual_layer_norm_kernel(float* __restri
     const int i = V * (threadIdx.x + k * NT);
 #pragma unroll
     for (int j = 0; j < V; ++j) v[k][j] = 0.f;
-    if (i < W) {
+    if (has_y && i < W) {
       if constexpr (V == 4) {
         const typename Vec4<Y>::type f = *reinterpret_cast<const typename Vec4<Y>::type*>(y + base + i);
 #pragma unroll
@@ -179,26 +197,43 @@ __global__ __launch_bounds__(NT) void residual_layer_norm_kernel(float* __restri
       }
     }
   }
-  float mean, r;
-  stats(eps, mean, r);
+  float mean = 0.f, r = 0.f;
+  if (has_y) stats(eps, mean, r);
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     const int i = V * (threadIdx.x + k * NT);
     if (i < W) {
       if constexpr (V == 4) {
         f32x4 x = *reinterpret_cast<const f32x4*>(resid + base + i);
-        const f32x4 pw = *reinterpret_cast<const f32x4*>(w + i), pb = *reinterpret_cast<const f32x4*>(b + i);
+        f32x4 pw = {0.f, 0.f, 0.f, 0.f}, pb = pw, en = pw;
+        if (has_y) pw = *reinterpret_cast<const f32x4*>(w + i);
+        if constexpr (LN) pb = *reinterpret_cast<const f32x4*>(b + i);
+        if (!LN && entry.add != nullptr) {
+          en = *reinterpret_cast<const f32x4*>(entry.add + i);
+          if (trow != nullptr) {
+            const typename Vec4<T>::type e = *reinterpret_cast<const typename Vec4<T>::type*>(trow + i);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) en[j] += Elem<T>::ld(e[j]);
+          }
+        }
         typename Vec4<T>::type o;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           x[j] += (v[k][j] - mean) * r * pw[j] + pb[j];
+          if constexpr (!LN) x[j] += en[j];
           v[k][j] = x[j];
           o[j] = Elem<T>::st(x[j]);
         }
         *reinterpret_cast<f32x4*>(resid + base + i) = x;
         if (pre_kind == 1) *reinterpret_cast<typename Vec4<T>::type*>(out + base + i) = o;
       } else {
-        const float x = resid[base + i] + (v[k][0] - mean) * r * w[i] + b[i];
+        float x = resid[base + i];
+        if constexpr (LN) {
+          x = x + (v[k][0] - mean) * r * w[i] + b[i];
+        } else {
+          if (has_y) x += v[k][0] * r * w[i];
+          if (entry.add != nullptr) x += entry.add[i] + (trow != nullptr ? Elem<T>::ld(trow[i]) : 0.f);
+        }
         v[k][0] = x;
         resid[base + i] = x;
         if (pre_kind == 1) out[base + i] = Elem<T>::st(x);
@@ -212,7 +247,17 @@ __global__ __launch_bounds__(NT) void residual_layer_norm_kernel(float* __restri
     const int i = V * (threadIdx.x + k * NT);
     if (i < W) {
 #pragma unroll
-      for (int j = 0; j < V; ++j) out[base + i + j] = Elem<T>::st((v[k][j] - mean) * r * qw[i + j] + qb[i + j]);
+      for (int j = 0; j < V; ++j) {
+        const float u = (v[k][j] - mean) * r * qw[i + j];
+        if constexpr (V == 4) v[k][j] = LN ? u + qb[i + j] : u;
+        else out[base + i + j] = Elem<T>::st(LN ? u + qb[i + j] : u);
+      }
+      if constexpr (V == 4) {
+        typename Vec4<T>::type o;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] = Elem<T>::st(v[k][j]);
+        *reinterpret_cast<typename Vec4<T>::type*>(out + base + i) = o;
+      }
     }
   }
 }
@@ -237,12 +282,12 @@ __global__ __launch_bounds__(NT) void rmsnorm_cols_kernel(const T* __restrict__ 
 // One wave per token (a row is a few hundred features: no block-wide reduction, four tokens per
 // workgroup).  Columns off .. off + R - 1 of the row are the latent (RMS norm, weight w),
 // the next RD the shared key part (the first 2 half of them turned by position * inv_freq, times
-// amp).  K slab of the token's page: features [latent | key part]; V^T slab: the latent.
+// amp; neighbours together with `pairs`).  K slab of the token's page: features [latent | key part]; V^T slab: the latent.
 template <typename T>
 __global__ __launch_bounds__(NT) void latent_kv_write_kernel(const T* __restrict__ y, int64_t stride, int off, int R, int RD,
                                                              const float* __restrict__ w, float eps,
                                                              const int* __restrict__ positions, const int* __restrict__ slots,
-                                                             const float* __restrict__ inv_freq, int half, float amp,
+                                                             const float* __restrict__ inv_freq, int half, float amp, int pairs,
                                                              T* __restrict__ k_cache, T* __restrict__ v_cache, int BS,
                                                              int num_blocks, int T_) {
   const int lane = threadIdx.x & 63;
@@ -274,13 +319,14 @@ __global__ __launch_bounds__(NT) void latent_kv_write_kernel(const T* __restrict
       const int j = i - R;
       val = Elem<T>::ld(row[i]);
       if (j < 2 * half) {
-        const int f = j < half ? j : j - half;
+        const bool first = pairs ? (j & 1) == 0 : j < half;   // of the two features that turn together
+        const int step = pairs ? 1 : half;
         float s, c;
-        sincosf(pos * inv_freq[f], &s, &c);
+        sincosf(pos * inv_freq[pairs ? j >> 1 : (first ? j : j - half)], &s, &c);
         s *= amp;
         c *= amp;
-        const float other = Elem<T>::ld(row[j < half ? i + half : i - half]);
-        val = j < half ? val * c - other * s : val * c + other * s;
+        const float other = Elem<T>::ld(row[first ? i + step : i - step]);
+        val = first ? val * c - other * s : val * c + other * s;
       }
     }
     if (swz) ks[(static_cast<size_t>(i >> 2) * BS + o) * 4 + (i & 3)] = Elem<T>::st(val);
@@ -289,13 +335,13 @@ __global__ __launch_bounds__(NT) void latent_kv_write_kernel(const T* __restrict
 }
 
 // dst[t, h, dst_off + j] = turn(src[t, h, src_off + j]), j < n: the first 2 half features of the
-// tail turn by position * inv_freq (j pairs with j + half), the others are copied.  A thread owns
+// tail turn by position * inv_freq (j pairs with j + half, or 2j with 2j + 1), the others are copied.  A thread owns
 // one pair (or one copied feature) of a token for `hpt` heads: with hpt = H one sincos serves all
 // heads of a token (large steps), with hpt = 1 every head has a thread of its own (small steps).
 template <typename T>
-__global__ __launch_bounds__(NT) void rope_half_tail_kernel(const T* __restrict__ src, int Ds, int src_off, T* __restrict__ dst,
+__global__ __launch_bounds__(NT) void rope_tail_kernel(const T* __restrict__ src, int Ds, int src_off, T* __restrict__ dst,
                                                             int Dd, int dst_off, int n, const int* __restrict__ positions,
-                                                            const float* __restrict__ inv_freq, int half, float amp,
+                                                            const float* __restrict__ inv_freq, int half, float amp, int pairs,
                                                             int64_t total, int H, int hpt) {
   const int per = n - half;   // work items of a (token, head chunk): `half` pairs, then the copied features
   const int chunks = H / hpt;
@@ -311,10 +357,11 @@ __global__ __launch_bounds__(NT) void rope_half_tail_kernel(const T* __restrict_
       sincosf(static_cast<float>(positions[t]) * inv_freq[j], &sn, &cs);
       sn *= amp;
       cs *= amp;
+      const int ia = pairs ? 2 * j : j, ib = pairs ? 2 * j + 1 : j + half;
       for (int h = 0; h < hpt; ++h) {
-        const float a = Elem<T>::ld(s[h * Ds + j]), b = Elem<T>::ld(s[h * Ds + j + half]);
-        d[h * Dd + j] = Elem<T>::st(a * cs - b * sn);
-        d[h * Dd + j + half] = Elem<T>::st(b * cs + a * sn);
+        const float a = Elem<T>::ld(s[h * Ds + ia]), b = Elem<T>::ld(s[h * Ds + ib]);
+        d[h * Dd + ia] = Elem<T>::st(a * cs - b * sn);
+        d[h * Dd + ib] = Elem<T>::st(b * cs + a * sn);
       }
     } else {
       for (int h = 0; h < hpt; ++h) d[h * Dd + j + half] = s[h * Ds + j + half];
@@ -370,10 +417,19 @@ __device__ __forceinline__ float gate_act(float z, int kind) {
   return kind == 0 ? siluf_arg(z, 1.5957691216057308f * (z + 0.044715f * z * z * z)) : siluf_(z);
 }
 
+// One gated hidden value from its two projections.  The activation of the gate is rounded as a
+// projection's output before the product, like every other activation; kind 3 (`clamped_glu`) rounds once.
+template <typename T>
+__device__ __forceinline__ T gated_value(float g, float u, int kind, float limit) {
+  if (kind == 3) return Elem<T>::st(clamped_glu(g, u, limit));
+  return Elem<T>::st(Elem<T>::ld(Elem<T>::st(gate_act(g, kind))) * u);
+}
+
 // out[r, c] = act(in[r, c]) * in[r, n + c], four columns per thread (n a multiple of 4, aligned):
 // blockIdx.y walks the rows.
 template <typename T>
-__global__ __launch_bounds__(NT) void gated_act_vec_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind) {
+__global__ __launch_bounds__(NT) void gated_act_vec_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind,
+                                                           float limit) {
   typedef typename Vec4<T>::type VT;
   const int c = 4 * (blockIdx.x * NT + threadIdx.x);
   if (c >= n) return;
@@ -381,7 +437,7 @@ __global__ __launch_bounds__(NT) void gated_act_vec_kernel(const T* __restrict__
     const VT g = *reinterpret_cast<const VT*>(in + r * 2 * n + c), u = *reinterpret_cast<const VT*>(in + r * 2 * n + n + c);
     VT o;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] = Elem<T>::st(Elem<T>::ld(Elem<T>::st(gate_act(Elem<T>::ld(g[j]), kind))) * Elem<T>::ld(u[j]));
+    for (int j = 0; j < 4; ++j) o[j] = gated_value<T>(Elem<T>::ld(g[j]), Elem<T>::ld(u[j]), kind, limit);
     *reinterpret_cast<VT*>(out + r * n + c) = o;
   }
 }
@@ -389,14 +445,13 @@ __global__ __launch_bounds__(NT) void gated_act_vec_kernel(const T* __restrict__
 // out[r, c] = act(in[r, c]) * in[r, n + c]: the hidden activation of a gated feed-forward from its
 // stacked [gate | up] projection.
 template <typename T>
-__global__ __launch_bounds__(NT) void gated_act_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind) {
+__global__ __launch_bounds__(NT) void gated_act_kernel(const T* __restrict__ in, T* __restrict__ out, int64_t rows, int n, int kind,
+                                                       float limit) {
   const int64_t total = rows * n;
   for (int64_t e = static_cast<int64_t>(blockIdx.x) * NT + threadIdx.x; e < total; e += static_cast<int64_t>(gridDim.x) * NT) {
     const int64_t r = e / n;
     const int c = static_cast<int>(e - r * n);
-    // rounded as a projection's output before the product, like every other activation
-    const float g = Elem<T>::ld(Elem<T>::st(gate_act(Elem<T>::ld(in[r * 2 * n + c]), kind)));
-    out[e] = Elem<T>::st(g * Elem<T>::ld(in[r * 2 * n + n + c]));
+    out[e] = gated_value<T>(Elem<T>::ld(in[r * 2 * n + c]), Elem<T>::ld(in[r * 2 * n + n + c]), kind, limit);
   }
 }
 
@@ -527,9 +582,10 @@ BCG_API int bcg_residual_layer_norm(void* resid, const void* y, int y_f32, const
               *qbf = static_cast<const float*>(qb);
   auto al16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
   const bool vec = W % 4 == 0 && al16(resid) && al16(y) && al16(out) && al16(w) && al16(b);
-#define BCG_RLN(TYPE, YTYPE, V, NV)                                                                                          \
-  residual_layer_norm_kernel<TYPE, YTYPE, V, NV><<<T_, NT, 0, s>>>(static_cast<float*>(resid), static_cast<const YTYPE*>(y), wf, \
-                                                                   bf, eps, pre_kind, qwf, qbf, pre_eps, static_cast<TYPE*>(out), W)
+  const StreamEntry entry{nullptr, nullptr, nullptr, 0};
+#define BCG_RLN(TYPE, YTYPE, V, NV)                                                                                              \
+  residual_row_norm_kernel<TYPE, YTYPE, V, NV, true><<<T_, NT, 0, s>>>(static_cast<float*>(resid), static_cast<const YTYPE*>(y), wf, \
+                                                                       bf, eps, pre_kind, qwf, qbf, pre_eps, static_cast<TYPE*>(out), W, entry)
 #define BCG_RLN_BY_WIDTH(TYPE, YTYPE)                                                    \
   do {                                                                                   \
     if (vec && W <= 4 * NT) BCG_RLN(TYPE, YTYPE, 4, 1);                                  \
@@ -540,6 +596,30 @@ BCG_API int bcg_residual_layer_norm(void* resid, const void* y, int y_f32, const
     else if (W <= 4 * NT) BCG_RLN(TYPE, YTYPE, 1, 4);                                    \
     else BCG_RLN(TYPE, YTYPE, 1, 64);                                                    \
   } while (0)
+  if (is_f32) BCG_RLN_BY_WIDTH(float, float);
+  else if (y_f32) BCG_RLN_BY_WIDTH(bf16_t, float);
+  else BCG_RLN_BY_WIDTH(bf16_t, bf16_t);
+#undef BCG_RLN
+  return BCG_CHECK_LAUNCH();
+}
+
+// x += rms(y) w (y null: nothing), then + add [W] + table[token] (add null: nothing; table null: only the
+// vector); pre_kind 0 / 1 / 2: nothing / rounded copy / RMS norm (qw, pre_eps) of the new x.  y_f32: y is
+// float whatever the activation type.  W <= 16384.
+BCG_API int bcg_residual_rms_norm(void* resid, const void* y, int y_f32, const void* w, float eps, const void* add,
+                                  const void* tokens, const void* table, int vocab, int pre_kind, const void* qw, float pre_eps,
+                                  void* out, int T_, int W, int is_f32, void* stream) {
+  if (T_ <= 0) return 0;
+  if (W < 1 || W > 16384 || pre_kind < 0 || pre_kind > 2 || (y != nullptr && w == nullptr) || (pre_kind == 2 && qw == nullptr)) return -2;
+  if (table != nullptr && (add == nullptr || tokens == nullptr || vocab < 1)) return -2;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const float *wf = static_cast<const float*>(w), *bf = nullptr, *qwf = static_cast<const float*>(qw), *qbf = nullptr;
+  auto al16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = W % 4 == 0 && al16(resid) && al16(y) && al16(out) && al16(w) && al16(add) && al16(table) && al16(qw);
+  const StreamEntry entry{static_cast<const float*>(add), static_cast<const int*>(tokens), table, vocab};
+#define BCG_RLN(TYPE, YTYPE, V, NV)                                                                                               \
+  residual_row_norm_kernel<TYPE, YTYPE, V, NV, false><<<T_, NT, 0, s>>>(static_cast<float*>(resid), static_cast<const YTYPE*>(y), wf, \
+                                                                        bf, eps, pre_kind, qwf, qbf, pre_eps, static_cast<TYPE*>(out), W, entry)
   if (is_f32) BCG_RLN_BY_WIDTH(float, float);
   else if (y_f32) BCG_RLN_BY_WIDTH(bf16_t, float);
   else BCG_RLN_BY_WIDTH(bf16_t, bf16_t);
@@ -559,7 +639,7 @@ BCG_API int bcg_rmsnorm_cols(const void* y, int64_t stride, int off, int n, cons
 }
 
 BCG_API int bcg_latent_kv_write(const void* y, int64_t stride, int off, int R, int RD, const void* w, float eps,
-                                const void* positions, const void* slots, const void* inv_freq, int half, float amp,
+                                const void* positions, const void* slots, const void* inv_freq, int half, float amp, int pairs,
                                 void* k_cache, void* v_cache, int T_, int BS, int num_blocks, int is_f32, void* stream) {
   if (T_ <= 0) return 0;
   if (R < 1 || RD < 0 || 2 * half > RD || BS % 16) return -2;
@@ -567,15 +647,15 @@ BCG_API int bcg_latent_kv_write(const void* y, int64_t stride, int off, int R, i
   const float *wf = static_cast<const float*>(w), *fr = static_cast<const float*>(inv_freq);
   const int *ps = static_cast<const int*>(positions), *sl = static_cast<const int*>(slots);
   const int grid = (T_ + NT / 64 - 1) / (NT / 64);
-  BCG_BY_TYPE((latent_kv_write_kernel<float><<<grid, NT, 0, s>>>(static_cast<const float*>(y), stride, off, R, RD, wf, eps, ps, sl, fr, half, amp,
+  BCG_BY_TYPE((latent_kv_write_kernel<float><<<grid, NT, 0, s>>>(static_cast<const float*>(y), stride, off, R, RD, wf, eps, ps, sl, fr, half, amp, pairs,
                                                                 static_cast<float*>(k_cache), static_cast<float*>(v_cache), BS, num_blocks, T_)),
-              (latent_kv_write_kernel<bf16_t><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(y), stride, off, R, RD, wf, eps, ps, sl, fr, half, amp,
+              (latent_kv_write_kernel<bf16_t><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(y), stride, off, R, RD, wf, eps, ps, sl, fr, half, amp, pairs,
                                                                  static_cast<bf16_t*>(k_cache), static_cast<bf16_t*>(v_cache), BS, num_blocks, T_)));
   return BCG_CHECK_LAUNCH();
 }
 
-BCG_API int bcg_rope_half_tail(const void* src, int Ds, int src_off, void* dst, int Dd, int dst_off, const void* positions,
-                               const void* inv_freq, int half, float amp, int T_, int H, int is_f32, void* stream) {
+BCG_API int bcg_rope_tail(const void* src, int Ds, int src_off, void* dst, int Dd, int dst_off, const void* positions,
+                               const void* inv_freq, int half, float amp, int pairs, int T_, int H, int is_f32, void* stream) {
   const int n = Ds - src_off;
   if (T_ <= 0 || H <= 0 || n <= 0) return 0;
   if (n != Dd - dst_off || 2 * half > n) return -2;
@@ -584,10 +664,10 @@ BCG_API int bcg_rope_half_tail(const void* src, int Ds, int src_off, void* dst, 
   const int64_t total = static_cast<int64_t>(T_) * (H / hpt) * (n - half);
   const int* ps = static_cast<const int*>(positions);
   const float* fr = static_cast<const float*>(inv_freq);
-  BCG_BY_TYPE((rope_half_tail_kernel<float><<<ew_grid(total), NT, 0, s>>>(static_cast<const float*>(src), Ds, src_off, static_cast<float*>(dst), Dd,
-                                                                         dst_off, n, ps, fr, half, amp, total, H, hpt)),
-              (rope_half_tail_kernel<bf16_t><<<ew_grid(total), NT, 0, s>>>(static_cast<const bf16_t*>(src), Ds, src_off, static_cast<bf16_t*>(dst), Dd,
-                                                                          dst_off, n, ps, fr, half, amp, total, H, hpt)));
+  BCG_BY_TYPE((rope_tail_kernel<float><<<ew_grid(total), NT, 0, s>>>(static_cast<const float*>(src), Ds, src_off, static_cast<float*>(dst), Dd,
+                                                                         dst_off, n, ps, fr, half, amp, pairs, total, H, hpt)),
+              (rope_tail_kernel<bf16_t><<<ew_grid(total), NT, 0, s>>>(static_cast<const bf16_t*>(src), Ds, src_off, static_cast<bf16_t*>(dst), Dd,
+                                                                          dst_off, n, ps, fr, half, amp, pairs, total, H, hpt)));
   return BCG_CHECK_LAUNCH();
 }
 
@@ -615,18 +695,19 @@ BCG_API int bcg_gate_mul(const void* x, const void* gate, int64_t gate_stride, v
   return BCG_CHECK_LAUNCH();
 }
 
-BCG_API int bcg_gated_act(const void* in, void* out, int64_t rows, int n, int kind, int is_f32, void* stream) {
+// kind 0 / 2: gelu / silu of the gate; 3: the clamped product with `limit`.
+BCG_API int bcg_gated_act(const void* in, void* out, int64_t rows, int n, int kind, float limit, int is_f32, void* stream) {
   if (rows <= 0 || n <= 0) return 0;
-  if (kind != 0 && kind != 2) return -2;
+  if (kind != 0 && kind != 2 && kind != 3) return -2;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (n % 4 == 0 && ((reinterpret_cast<uintptr_t>(in) | reinterpret_cast<uintptr_t>(out)) & 15) == 0) {
     const dim3 grid((n / 4 + NT - 1) / NT, static_cast<unsigned>(std::min<int64_t>(rows, 65535)));
-    BCG_BY_TYPE((gated_act_vec_kernel<float><<<grid, NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind)),
-                (gated_act_vec_kernel<bf16_t><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind)));
+    BCG_BY_TYPE((gated_act_vec_kernel<float><<<grid, NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind, limit)),
+                (gated_act_vec_kernel<bf16_t><<<grid, NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind, limit)));
     return BCG_CHECK_LAUNCH();
   }
-  BCG_BY_TYPE((gated_act_kernel<float><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind)),
-              (gated_act_kernel<bf16_t><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind)));
+  BCG_BY_TYPE((gated_act_kernel<float><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const float*>(in), static_cast<float*>(out), rows, n, kind, limit)),
+              (gated_act_kernel<bf16_t><<<ew_grid(rows * n), NT, 0, s>>>(static_cast<const bf16_t*>(in), static_cast<bf16_t*>(out), rows, n, kind, limit)));
   return BCG_CHECK_LAUNCH();
 }
 

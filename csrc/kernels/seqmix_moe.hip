@@ -132,15 +132,22 @@ __global__ __launch_bounds__(1024) void align_kernel(const int* __restrict__ idx
   }
 }
 
-// Epilogue of a gated expert's first product (act 2).  The N rows of the expert's weight are its
+// Hidden value of a gated expert from its two products (rounded to T like a projection's output):
+// act 2 silu(gate) * up, the activation rounded too; act 3 `clamped_glu`, rounded once.
+template <typename T>
+__device__ __forceinline__ T gated_hidden(float gate, float up, int act, float limit) {
+  const float g = Elem<T>::ld(Elem<T>::st(gate)), u = Elem<T>::ld(Elem<T>::st(up));
+  if (act == 3) return Elem<T>::st(clamped_glu(g, u, limit));
+  return Elem<T>::st(Elem<T>::ld(Elem<T>::st(g / (1.0f + expf(-g)))) * u);
+}
+
+// Epilogue of a gated expert's first product (act 2, 3).  The N rows of the expert's weight are its
 // gate and up rows in alternating groups of 16 ([gate 0..15 | up 0..15 | gate 16..31 | ...]), so a
 // wave's n tiles 0 / 2 hold gate columns and tiles 1 / 3 the up columns of the SAME features:
-// out[r, f] = silu(gate_f) * up_f with f = n / 2 (N / 2 output columns), both factors and the
-// activation rounded to T like a projection's output.
+// out[r, f] = gated_hidden(gate_f, up_f) with f = n / 2 (N / 2 output columns).
 template <typename T>
 __device__ __forceinline__ void store_gated(const f32x4 (&acc)[4][4], const int (&slot)[4], T* __restrict__ out,
-                                            int64_t out_stride, int scatter, int p0, int n0, int N, int col, int grp) {
-  auto rnd = [](float v) { return Elem<T>::ld(Elem<T>::st(v)); };
+                                            int64_t out_stride, int scatter, int p0, int n0, int N, int col, int grp, int act, float limit) {
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     if (slot[j] < 0) continue;
@@ -149,22 +156,21 @@ __device__ __forceinline__ void store_gated(const f32x4 (&acc)[4][4], const int 
     for (int i2 = 0; i2 < 2; ++i2)
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        if (n0 + 32 * i2 + 16 + 4 * grp + q < N) {
-          const float g = rnd(acc[2 * i2][j][q]), u = rnd(acc[2 * i2 + 1][j][q]);
-          out[r * out_stride + (n0 >> 1) + 16 * i2 + 4 * grp + q] = Elem<T>::st(rnd(g / (1.0f + expf(-g))) * u);
-        }
+        if (n0 + 32 * i2 + 16 + 4 * grp + q < N)
+          out[r * out_stride + (n0 >> 1) + 16 * i2 + 4 * grp + q] =
+              gated_hidden<T>(acc[2 * i2][j][q], acc[2 * i2 + 1][j][q], act, limit);
       }
   }
 }
 
 // Position p of tile blockIdx.x: slot = sorted[p] (-1: padding).  gather: A row = a[(slot / top)]
-// (token rows), else a[p].  scatter: output row = slot, else p.  act 1: relu squared; act 2: `store_gated`.
+// (token rows), else a[p].  scatter: output row = slot, else p.  act 1: relu squared; act 2, 3: `store_gated`.
 template <typename T, bool FULL>
 __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ a, int64_t a_stride, const T* __restrict__ w,
                                                        T* __restrict__ out, int64_t out_stride,
                                                        const int* __restrict__ sorted,
                                                        const int* __restrict__ tile_expert, int N, int K, int top,
-                                                       int gather, int scatter, int act, int vec) {
+                                                       int gather, int scatter, int act, float limit, int vec) {
   typedef typename Elem<T>::frag F;
   const int e = tile_expert[blockIdx.x];
   if (e < 0) return;
@@ -205,8 +211,8 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ a, 
 #pragma unroll
       for (int j = 0; j < 4; ++j) acc[i][j] = mma16(wf[i], af[j], acc[i][j]);
   }
-  if (act == 2) {
-    store_gated<T>(acc, slot, out, out_stride, scatter, p0, n0, N, col, grp);
+  if (act >= 2) {
+    store_gated<T>(acc, slot, out, out_stride, scatter, p0, n0, N, col, grp, act, limit);
     return;
   }
 #pragma unroll
@@ -237,7 +243,7 @@ __global__ __launch_bounds__(256) void moe_gemm_lds_kernel(const T* __restrict__
                                                            T* __restrict__ out, int64_t out_stride,
                                                            const int* __restrict__ sorted,
                                                            const int* __restrict__ tile_expert, int N, int K, int top,
-                                                           int gather, int scatter, int act) {
+                                                           int gather, int scatter, int act, float limit) {
   typedef typename Elem<T>::frag F;
   constexpr int BK = 32, LDK = BK + 8;   // rows stay 16-byte aligned for the 8-element fragment reads
   typedef T Chunk __attribute__((ext_vector_type(8)));   // 8 consecutive elements (16 or 32 bytes)
@@ -320,8 +326,8 @@ __global__ __launch_bounds__(256) void moe_gemm_lds_kernel(const T* __restrict__
     }
   }
   const int n0 = nb + 64 * wave;
-  if (act == 2) {
-    store_gated<T>(acc, slot, out, out_stride, scatter, p0, n0, N, col, grp);
+  if (act >= 2) {
+    store_gated<T>(acc, slot, out, out_stride, scatter, p0, n0, N, col, grp, act, limit);
     return;
   }
 #pragma unroll
@@ -350,7 +356,7 @@ __global__ __launch_bounds__(256) void moe_gemm_lds_narrow_kernel(const T* __res
                                                                   const T* __restrict__ w, T* __restrict__ out,
                                                                   int64_t out_stride, const int* __restrict__ sorted,
                                                                   const int* __restrict__ tile_expert, int N, int K, int top,
-                                                                  int gather, int scatter, int act) {
+                                                                  int gather, int scatter, int act, float limit) {
   typedef typename Elem<T>::frag F;
   constexpr int BK = 32, LDK = BK + 8, TNN = 64;
   typedef T Chunk __attribute__((ext_vector_type(8)));
@@ -409,16 +415,13 @@ __global__ __launch_bounds__(256) void moe_gemm_lds_narrow_kernel(const T* __res
   }
   if (slot < 0) return;
   const int64_t r = scatter ? slot : p0 + 16 * wave + col;
-  if (act == 2) {   // gate / up column pairs, as `store_gated`
-    auto rnd = [](float v) { return Elem<T>::ld(Elem<T>::st(v)); };
+  if (act >= 2) {   // gate / up column pairs, as `store_gated`
 #pragma unroll
     for (int i2 = 0; i2 < 2; ++i2)
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        if (nb + 32 * i2 + 16 + 4 * grp + q < N) {
-          const float g = rnd(acc[2 * i2][q]), u = rnd(acc[2 * i2 + 1][q]);
-          out[r * out_stride + (nb >> 1) + 16 * i2 + 4 * grp + q] = Elem<T>::st(rnd(g / (1.0f + expf(-g))) * u);
-        }
+        if (nb + 32 * i2 + 16 + 4 * grp + q < N)
+          out[r * out_stride + (nb >> 1) + 16 * i2 + 4 * grp + q] = gated_hidden<T>(acc[2 * i2][q], acc[2 * i2 + 1][q], act, limit);
       }
     return;
   }
@@ -496,16 +499,16 @@ BCG_API int bcg_moe_align(const void* idx, int n_slots, int E, void* sorted, int
 
 BCG_API int bcg_moe_gemm(const void* a, int64_t a_stride, const void* w, void* out, int64_t out_stride, const void* sorted,
                          const void* tile_expert, int n_tiles, int N, int K, int top, int gather, int scatter, int act,
-                         int is_f32, void* stream) {
+                         float limit, int is_f32, void* stream) {
   if (n_tiles <= 0) return 0;
-  if (N < 1 || K < 1 || n_tiles > (1 << 24) || (N + TN - 1) / TN > 65535 || (act == 2 && N % 32)) return -2;
+  if (N < 1 || K < 1 || n_tiles > (1 << 24) || (N + TN - 1) / TN > 65535 || act < 0 || act > 3 || (act >= 2 && N % 32)) return -2;
   hipStream_t s = static_cast<hipStream_t>(stream);
   dim3 grid(n_tiles, (N + TN - 1) / TN);
   const int vec = (K % 4 == 0 && a_stride % 4 == 0) ? 1 : 0;
 #define BCG_MOE_GEMM(TYPE, FULL_)                                                                                    \
   moe_gemm_kernel<TYPE, FULL_><<<grid, 256, 0, s>>>(static_cast<const TYPE*>(a), a_stride, static_cast<const TYPE*>(w), \
                                                     static_cast<TYPE*>(out), out_stride, static_cast<const int*>(sorted), \
-                                                    static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, vec)
+                                                    static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, limit, vec)
   const bool full = vec && K % 16 == 0;   // whole, aligned fragments only
   const int esz = is_f32 ? 4 : 2;
   if (K % 32 == 0 && (a_stride * esz) % 16 == 0 && (reinterpret_cast<uintptr_t>(a) | reinterpret_cast<uintptr_t>(w)) % 16 == 0) {
@@ -514,21 +517,21 @@ BCG_API int bcg_moe_gemm(const void* a, int64_t a_stride, const void* w, void* o
       if (is_f32)
         moe_gemm_lds_narrow_kernel<float><<<ngrid, 256, 0, s>>>(static_cast<const float*>(a), a_stride, static_cast<const float*>(w),
                                                                static_cast<float*>(out), out_stride, static_cast<const int*>(sorted),
-                                                               static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act);
+                                                               static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, limit);
       else
         moe_gemm_lds_narrow_kernel<bf16_t><<<ngrid, 256, 0, s>>>(static_cast<const bf16_t*>(a), a_stride, static_cast<const bf16_t*>(w),
                                                                 static_cast<bf16_t*>(out), out_stride, static_cast<const int*>(sorted),
-                                                                static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act);
+                                                                static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, limit);
       return BCG_CHECK_LAUNCH();
     }
     if (is_f32)
       moe_gemm_lds_kernel<float><<<grid, 256, 0, s>>>(static_cast<const float*>(a), a_stride, static_cast<const float*>(w),
                                                      static_cast<float*>(out), out_stride, static_cast<const int*>(sorted),
-                                                     static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act);
+                                                     static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, limit);
     else
       moe_gemm_lds_kernel<bf16_t><<<grid, 256, 0, s>>>(static_cast<const bf16_t*>(a), a_stride, static_cast<const bf16_t*>(w),
                                                       static_cast<bf16_t*>(out), out_stride, static_cast<const int*>(sorted),
-                                                      static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act);
+                                                      static_cast<const int*>(tile_expert), N, K, top, gather, scatter, act, limit);
     return BCG_CHECK_LAUNCH();
   }
   if (is_f32) {

@@ -21,9 +21,11 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return t;
 }
 
+// x = table[token] * scale (+ add, one vector for all rows), out = norm(x).
 template <typename T>
 __global__ __launch_bounds__(NT) void embed_scale_norm_kernel(const int* __restrict__ tokens, const T* __restrict__ table,
-                                                              float scale, const float* __restrict__ w, float eps,
+                                                              float scale, const float* __restrict__ add,
+                                                              const float* __restrict__ w, float eps,
                                                               float w_offset, float* __restrict__ resid,
                                                               T* __restrict__ out, int W, int vocab) {
   __shared__ float red[NT / 64];
@@ -34,7 +36,8 @@ __global__ __launch_bounds__(NT) void embed_scale_norm_kernel(const int* __restr
   float* x = resid + static_cast<size_t>(t) * W;
   float ss = 0.f;
   for (int i = threadIdx.x; i < W; i += NT) {
-    const float v = Elem<T>::ld(row[i]) * scale;
+    float v = Elem<T>::ld(row[i]) * scale;
+    if (add != nullptr) v += add[i];
     x[i] = v;
     ss += v * v;
   }
@@ -188,17 +191,17 @@ __global__ __launch_bounds__(NT) void rope_multi_kv_kernel(const T* __restrict__
 
 }  // namespace
 
-BCG_API int bcg_embed_scale_rmsnorm(const void* tokens, const void* table, float scale, const void* w, float eps,
+BCG_API int bcg_embed_scale_rmsnorm(const void* tokens, const void* table, float scale, const void* add, const void* w, float eps,
                                     float w_offset, void* resid, void* out, int T_, int W, int vocab, int is_f32,
                                     void* stream) {
   if (T_ <= 0) return 0;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (is_f32)
-    embed_scale_norm_kernel<float><<<T_, NT, 0, s>>>(static_cast<const int*>(tokens), static_cast<const float*>(table), scale,
+    embed_scale_norm_kernel<float><<<T_, NT, 0, s>>>(static_cast<const int*>(tokens), static_cast<const float*>(table), scale, static_cast<const float*>(add),
                                                     static_cast<const float*>(w), eps, w_offset,
                                                     static_cast<float*>(resid), static_cast<float*>(out), W, vocab);
   else
-    embed_scale_norm_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const int*>(tokens), static_cast<const bf16_t*>(table), scale,
+    embed_scale_norm_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const int*>(tokens), static_cast<const bf16_t*>(table), scale, static_cast<const float*>(add),
                                                      static_cast<const float*>(w), eps, w_offset,
                                                      static_cast<float*>(resid), static_cast<bf16_t*>(out), W, vocab);
   return BCG_CHECK_LAUNCH();

@@ -20,7 +20,7 @@ namespace {
 constexpr int NT = 256;
 constexpr int MAX_TAPS = 16;
 constexpr int SCAN_CHUNK_ELEMS = 512;   // rows x tokens of a recurrence staged through LDS at a time
-constexpr int SCAN_WAVES = 4;   // waves of a recurrence workgroup (8 value columns each)   // tokens of a recurrence staged through LDS at a time
+constexpr int SCAN_WAVES = 4;   // waves of a recurrence workgroup (8 value columns each)
 
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);
@@ -271,7 +271,7 @@ __global__ __launch_bounds__(NT) void short_conv_state_kernel(const T* __restric
 // ---------------------------------------------------------------- whole-projection norms, pair rotary, rotated values
 // One block per token.  Row [q (n_q dim) | k (n_kv dim) | v (n_kv vdim) | ...].  q and k are each
 // RMS-normed over their whole width (weights q_norm / k_norm; null = as they are); features
-// (2i, 2i + 1), i < half, of every q / k head turn by position * inv_freq[i]; every pair of every v
+// (2i, 2i + 1), i < half, of every q / k head turn by position * inv_freq[i], cos and sin times amp; every pair of every v
 // head by position * v_inv_freq[i] (null = as they are).  K / V^T go to the paged cache in the
 // slab layout of seqmix_attention.hip (one map).  The values start at column v_off (at the k part
 // itself when the values are the keys before their norm); q is also multiplied by its temperature.
@@ -279,7 +279,7 @@ template <typename T>
 __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__ qkv, int64_t row_stride,
                                                            const int* __restrict__ positions, const int* __restrict__ slots,
                                                            const float* __restrict__ q_norm, const float* __restrict__ k_norm,
-                                                           float eps, const float* __restrict__ inv_freq, int half,
+                                                           float eps, const float* __restrict__ inv_freq, int half, float amp,
                                                            const float* __restrict__ v_inv_freq, T* __restrict__ q_out,
                                                            T* __restrict__ k_cache, T* __restrict__ v_cache, int n_q, int n_kv,
                                                            int dim, int vdim, int v_off, float temp_coef, int temp_every,
@@ -322,6 +322,8 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
       const float other = Elem<T>::ld(row[idx ^ 1]) * rn * (wn != nullptr ? wn[wi ^ 1] : 1.0f);
       float s, c;
       sincosf(pos * inv_freq[i >> 1], &s, &c);
+      s *= amp;
+      c *= amp;
       val = (i & 1) ? val * c + other * s : val * c - other * s;
     }
     if (is_q) {
@@ -351,30 +353,49 @@ __global__ __launch_bounds__(NT) void rope_pairs_kv_kernel(const T* __restrict__
   }
 }
 
-// The same without any rotation (half = 0, values as they are), four features per access: dim, vdim,
-// the row stride and the row's start are multiples of four elements.  TPB tokens per workgroup:
+// The same with values as they are, four features per access: dim, vdim,
+// the row stride and the row's start are multiples of four elements.  ROT: the q / k heads turn; a
+// token's cosines and sines are computed once into LDS (dim / 2 pairs, 1 and 0 past `half`) and serve
+// all its heads.  TPB tokens per workgroup:
 // 4 (a wave per token; four tokens on consecutive slots of one 4-key group write their values as
 // whole groups) for large steps, 1 for small ones.
-template <typename T, int TPB>
+constexpr int ROT_PAIRS = 256;   // pairs of a head in the LDS table (dim <= 512)
+
+template <typename T, int TPB, bool ROT>
 __global__ __launch_bounds__(NT) void norm_kv_kernel(const T* __restrict__ qkv, int64_t row_stride, const int* __restrict__ positions,
                                                      const int* __restrict__ slots, const float* __restrict__ q_norm,
-                                                     const float* __restrict__ k_norm, float eps, T* __restrict__ q_out,
+                                                     const float* __restrict__ k_norm, float eps,
+                                                     const float* __restrict__ inv_freq, int half, float amp, T* __restrict__ q_out,
                                                      T* __restrict__ k_cache, T* __restrict__ v_cache, int n_q, int n_kv, int dim,
                                                      int vdim, int v_off, float temp_coef, int temp_every, int BS, int num_blocks,
                                                      int n_tokens) {
   typedef typename Elem<T>::frag F;
   constexpr int TPT = NT / TPB;   // threads per token
   __shared__ float red[2][NT / 64];
+  __shared__ float table[ROT ? TPB : 1][ROT ? 2 * ROT_PAIRS : 2];   // cosines, then sines
   const int sub = threadIdx.x / TPT, tid = threadIdx.x - sub * TPT;
   const int t = blockIdx.x * TPB + sub;
   const bool live = t < n_tokens;
+  if constexpr (ROT) {
+    const float pos = static_cast<float>(positions[live ? t : n_tokens - 1]);
+    for (int i = tid; i < (dim >> 1); i += TPT) {
+      float s = 0.f, c = 1.f;
+      if (i < half) {
+        sincosf(pos * inv_freq[i], &s, &c);
+        s *= amp;
+        c *= amp;
+      }
+      table[sub][i] = c;
+      table[sub][ROT_PAIRS + i] = s;
+    }
+  }
   const int qw = n_q * dim, kw = n_kv * dim, vw = n_kv * vdim;
   const T* row = qkv + static_cast<size_t>(live ? t : n_tokens - 1) * row_stride;
   auto get = [](const F& f, int j) {
     if constexpr (sizeof(T) == 2) return bf2f(static_cast<bf16_t>(f[j])); else return f[j];
   };
   float sq = 0.f, sk = 0.f;
-  for (int i = 4 * tid; i < qw + kw; i += 4 * TPT) {
+  if (q_norm != nullptr || k_norm != nullptr) for (int i = 4 * tid; i < qw + kw; i += 4 * TPT) {
     const F f = *reinterpret_cast<const F*>(row + i);
     float s = 0.f;
 #pragma unroll
@@ -383,6 +404,7 @@ __global__ __launch_bounds__(NT) void norm_kv_kernel(const T* __restrict__ qkv, 
   }
   sq = wave_sum(sq);
   sk = wave_sum(sk);
+  if constexpr (ROT && TPB > 1) __syncthreads();   // the tables
   if constexpr (TPB == 1) {
     if ((threadIdx.x & 63) == 0) {
       red[0][threadIdx.x >> 6] = sq;
@@ -411,10 +433,22 @@ __global__ __launch_bounds__(NT) void norm_kv_kernel(const T* __restrict__ qkv, 
       f32x4 w = {1.f, 1.f, 1.f, 1.f};
       if (wn != nullptr) w = *reinterpret_cast<const f32x4*>(wn + wi);
       const float r = is_q ? rq : rk;
+      float v[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = get(f, j) * r * w[j];
+      if constexpr (ROT) {
+        const int pair = (wi % dim) >> 1;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          const float c = table[sub][pair + j], s = table[sub][ROT_PAIRS + pair + j], a = v[2 * j], b = v[2 * j + 1];
+          v[2 * j] = a * c - b * s;
+          v[2 * j + 1] = b * c + a * s;
+        }
+      }
       F o;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const T e = Elem<T>::st(get(f, j) * r * w[j]);
+        const T e = Elem<T>::st(v[j]);
         if constexpr (sizeof(T) == 2) o[j] = static_cast<short>(e); else o[j] = e;
       }
       if (is_q) {
@@ -498,6 +532,75 @@ __global__ __launch_bounds__(NT) void hgrn2_prepare_kernel(const T* __restrict__
   }
 }
 
+// Retention.  One block per token: the heads of two column blocks (q at off_q, k at off_k, n_heads x dim
+// each) turned by the position (feature i pairs with i + half, cos and sin times amp), k also times
+// k_scale, as fp32.  VEC: four pairs per access (half, dim and the row's start multiples of four).
+template <typename T, bool VEC>
+__global__ __launch_bounds__(NT) void retention_prepare_kernel(const T* __restrict__ y, int64_t stride, int off_q, int off_k,
+                                                               int n_heads, int dim, const int* __restrict__ positions,
+                                                               const float* __restrict__ inv_freq, int half, float amp, float k_scale,
+                                                               float* __restrict__ q32, float* __restrict__ k32) {
+  extern __shared__ float table[];   // [half] cosines, [half] sines
+  typedef typename Elem<T>::frag F;
+  constexpr int V = VEC ? 4 : 1;
+  const int t = blockIdx.x;
+  const float pos = static_cast<float>(positions[t]);
+  for (int i = threadIdx.x; i < half; i += NT) {
+    float s, c;
+    sincosf(pos * inv_freq[i], &s, &c);
+    table[i] = c * amp;
+    table[half + i] = s * amp;
+  }
+  __syncthreads();
+  const T* row = y + static_cast<size_t>(t) * stride;
+  const size_t obase = static_cast<size_t>(t) * n_heads * dim;
+  const int turned = half / V, per = turned + (dim - 2 * half) / V;   // work items of a head: turned pairs, then plain features
+  auto load = [&](const T* p, float (&v)[V]) {
+    if constexpr (VEC) {
+      const F f = *reinterpret_cast<const F*>(p);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if constexpr (sizeof(T) == 2) v[j] = bf2f(static_cast<bf16_t>(f[j])); else v[j] = f[j];
+      }
+    } else {
+      v[0] = Elem<T>::ld(*p);
+    }
+  };
+  auto store = [&](float* p, const float (&v)[V]) {
+    if constexpr (VEC) *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
+    else *p = v[0];
+  };
+  for (int item = threadIdx.x; item < 2 * n_heads * per; item += NT) {
+    const int vh = item / per, c = item - vh * per;
+    const bool is_q = vh < n_heads;
+    const int h = is_q ? vh : vh - n_heads;
+    const T* src = row + (is_q ? off_q : off_k) + h * dim;
+    float* dst = (is_q ? q32 : k32) + obase + static_cast<size_t>(h) * dim;
+    const float sc = is_q ? 1.0f : k_scale;
+    if (c < turned) {
+      const int i = V * c;
+      float a[V], b[V], ra[V], rb[V];
+      load(src + i, a);
+      load(src + i + half, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float cs = table[i + j], sn = table[half + i + j];
+        ra[j] = (a[j] * cs - b[j] * sn) * sc;
+        rb[j] = (b[j] * cs + a[j] * sn) * sc;
+      }
+      store(dst + i, ra);
+      store(dst + i + half, rb);
+    } else {
+      const int i = 2 * half + V * (c - turned);
+      float a[V];
+      load(src + i, a);
+#pragma unroll
+      for (int j = 0; j < V; ++j) a[j] *= sc;
+      store(dst + i, a);
+    }
+  }
+}
+
 // Gated delta rule.  One block per token: q / k heads (G of them, from the convolved row c) become
 // unit vectors x / sqrt(sum x^2 + 1e-6), q also times dim^-1/2; beta = sigmoid(y[off_beta + h]);
 // decay g[h, i] = exp(-exp(a_log[h]) softplus(a[h, i] + dt_bias[h, i])), i < gd: gd = dim (a decay per
@@ -536,7 +639,8 @@ __global__ __launch_bounds__(NT) void delta_prepare_kernel(const T* __restrict__
 // ---------------------------------------------------------------- the recurrence
 // Per head a dim x vdim fp32 state S; token after token
 //     S <- diag(g_t) S;  u = DELTA ? beta_t (v_t - S^T k_t) : beta_t v_t;  S <- S + k_t u^T;  o_t = S^T q_t
-// (beta null without DELTA: u = v_t; gd = 1: g_t is one number per head, else one per key channel).
+// (beta null without DELTA: u = v_t; gd = 1: g_t is one number per head, else one per key channel;
+// g_token = 0: the same decays for every token).
 // One workgroup of SCAN_WAVES waves per (segment, head, 8 SCAN_WAVES value columns); a wave owns 8
 // columns: lane = 8 column + row group, so a lane keeps
 // dim / 8 rows of one column of S in registers and the two sums over rows (S^T k and S^T q) are
@@ -555,7 +659,7 @@ struct ScanArgs {
   const int* positions; const int* q_start; const int* state_rows;
   float* state;                                     // [n_rows, H, dim, vdim]
   float* out;                                       // [T, H, vdim]
-  int n_rows, H, Gq, dim, vdim, gd;
+  int n_rows, H, Gq, dim, vdim, gd, g_token;        // g_token: elements of g per token, H gd or 0
 };
 
 template <int CTRL>
@@ -608,9 +712,9 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void state_scan_kernel(ScanArgs a)
     src_ok[n] = which < 3 && i < dim;
     const float* p = which == 0 ? a.q + (static_cast<size_t>(t0) * a.Gq + gq) * dim
                    : which == 1 ? a.k + (static_cast<size_t>(t0) * a.Gq + gq) * dim
-                                : a.g + (static_cast<size_t>(t0) * a.H + h) * a.gd;
+                                : a.g + static_cast<size_t>(t0) * a.g_token + h * a.gd;
     src[n] = p + ((src_ok[n] && (which < 2 || a.gd > 1)) ? i : 0);
-    step[n] = which < 2 ? static_cast<int64_t>(a.Gq) * dim : static_cast<int64_t>(a.H) * a.gd;
+    step[n] = which < 2 ? static_cast<int64_t>(a.Gq) * dim : a.g_token;
   }
   const T* vsrc = vbase + static_cast<size_t>(t0) * a.v_stride;
   const bool scaled = a.beta != nullptr;   // (always with DELTA)
@@ -711,7 +815,7 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void state_scan_kernel(ScanArgs a)
 }
 
 // o fp32 [T, H, vdim] -> out [T, H vdim]: every head over its root mean square, times w [vdim]
-// (w_head = 0) or w [H vdim] (w_head = vdim), times sigmoid(gate[t, h vdim + e]) (gate_kind 0) or silu
+// (w_head = 0) or w [H vdim] (w_head = vdim) (null: no weight), times sigmoid(gate[t, h vdim + e]) (gate_kind 0) or silu
 // of it (1) (gate null: none).  With `floor_` [T, H] a head of o has vdim + 1 columns and is first
 // divided by max(|last column|, floor) + 1e-6 (a memory read beside its normaliser).  One wave per
 // (token, head).
@@ -731,7 +835,8 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restr
   const int64_t t = th / H;
   const int h = static_cast<int>(th - t * H);
   for (int e = lane; e < vdim; e += 64) {
-    float v = x[e] * r * w[h * w_head + e];
+    float v = x[e] * r;
+    if (w != nullptr) v *= w[h * w_head + e];
     if (gate != nullptr) {
       const float z = Elem<T>::ld(gate[t * gate_stride + static_cast<int64_t>(h) * vdim + e]);
       v *= gate_kind == 0 ? sigmoidf_(z) : z * sigmoidf_(z);
@@ -826,7 +931,7 @@ BCG_API int bcg_short_conv(const void* y, int64_t y_stride, int C, const void* w
 }
 
 BCG_API int bcg_rope_pairs_kv_write(const void* qkv, int64_t row_stride, const void* positions, const void* slots,
-                                    const void* q_norm, const void* k_norm, float eps, const void* inv_freq, int half,
+                                    const void* q_norm, const void* k_norm, float eps, const void* inv_freq, int half, float amp,
                                     const void* v_inv_freq, void* q_out, void* k_cache, void* v_cache, int T_, int n_q,
                                     int n_kv, int dim, int vdim, int v_off, float temp_coef, int temp_every, int BS,
                                     int num_blocks, int is_f32, void* stream) {
@@ -838,23 +943,28 @@ BCG_API int bcg_rope_pairs_kv_write(const void* qkv, int64_t row_stride, const v
   const float *qn = static_cast<const float*>(q_norm), *kn = static_cast<const float*>(k_norm),
               *fr = static_cast<const float*>(inv_freq), *vf = static_cast<const float*>(v_inv_freq);
   auto al = [](const void* q, int b) { return (reinterpret_cast<uintptr_t>(q) & (b - 1)) == 0; };
-  if (half == 0 && vf == nullptr && dim % 4 == 0 && vdim % 4 == 0 && row_stride % 4 == 0 && al(qkv, is_f32 ? 16 : 8) && al(q_out, 16) &&
+  if ((half == 0 || dim <= 2 * ROT_PAIRS) && vf == nullptr && dim % 4 == 0 && vdim % 4 == 0 && row_stride % 4 == 0 && al(qkv, is_f32 ? 16 : 8) && al(q_out, 16) &&
       al(k_cache, 16) && al(v_cache, 16) && al(qn, 16) && al(kn, 16)) {
-#define BCG_NORM_KV(TYPE, TPB)                                                                                                    \
-  norm_kv_kernel<TYPE, TPB><<<(T_ + TPB - 1) / TPB, NT, 0, s>>>(static_cast<const TYPE*>(qkv), row_stride, ps, sl, qn, kn, eps,  \
-                                                                static_cast<TYPE*>(q_out), static_cast<TYPE*>(k_cache),          \
-                                                                static_cast<TYPE*>(v_cache), n_q, n_kv, dim, vdim, v_off,        \
-                                                                temp_coef, temp_every, BS, num_blocks, T_)
-    if (T_ >= 1024) BCG_BY_TYPE((BCG_NORM_KV(float, 4)), (BCG_NORM_KV(bf16_t, 4)));
-    else BCG_BY_TYPE((BCG_NORM_KV(float, 1)), (BCG_NORM_KV(bf16_t, 1)));
+#define BCG_NORM_KV(TYPE, TPB, ROT)                                                                                                   \
+  norm_kv_kernel<TYPE, TPB, ROT><<<(T_ + TPB - 1) / TPB, NT, 0, s>>>(static_cast<const TYPE*>(qkv), row_stride, ps, sl, qn, kn, eps, \
+                                                                     fr, half, amp, static_cast<TYPE*>(q_out),                       \
+                                                                     static_cast<TYPE*>(k_cache), static_cast<TYPE*>(v_cache), n_q,  \
+                                                                     n_kv, dim, vdim, v_off, temp_coef, temp_every, BS, num_blocks, T_)
+    if (half == 0) {
+      if (T_ >= 1024) BCG_BY_TYPE((BCG_NORM_KV(float, 4, false)), (BCG_NORM_KV(bf16_t, 4, false)));
+      else BCG_BY_TYPE((BCG_NORM_KV(float, 1, false)), (BCG_NORM_KV(bf16_t, 1, false)));
+    } else {
+      if (T_ >= 1024) BCG_BY_TYPE((BCG_NORM_KV(float, 4, true)), (BCG_NORM_KV(bf16_t, 4, true)));
+      else BCG_BY_TYPE((BCG_NORM_KV(float, 1, true)), (BCG_NORM_KV(bf16_t, 1, true)));
+    }
 #undef BCG_NORM_KV
     return BCG_CHECK_LAUNCH();
   }
-  BCG_BY_TYPE((rope_pairs_kv_kernel<float><<<T_, NT, 0, s>>>(static_cast<const float*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half,
+  BCG_BY_TYPE((rope_pairs_kv_kernel<float><<<T_, NT, 0, s>>>(static_cast<const float*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half, amp,
                                                             vf, static_cast<float*>(q_out), static_cast<float*>(k_cache),
                                                             static_cast<float*>(v_cache), n_q, n_kv, dim, vdim, v_off, temp_coef, temp_every, BS,
                                                             num_blocks)),
-              (rope_pairs_kv_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const bf16_t*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half,
+              (rope_pairs_kv_kernel<bf16_t><<<T_, NT, 0, s>>>(static_cast<const bf16_t*>(qkv), row_stride, ps, sl, qn, kn, eps, fr, half, amp,
                                                              vf, static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_cache),
                                                              static_cast<bf16_t*>(v_cache), n_q, n_kv, dim, vdim, v_off, temp_coef, temp_every, BS,
                                                              num_blocks)));
@@ -891,6 +1001,27 @@ BCG_API int bcg_hgrn2_prepare(const void* y, int64_t stride, int off_q, int off_
   return BCG_CHECK_LAUNCH();
 }
 
+BCG_API int bcg_retention_prepare(const void* y, int64_t stride, int off_q, int off_k, int n_heads, int dim, const void* positions,
+                                  const void* inv_freq, int half, float amp, float k_scale, void* q32, void* k32, int T_, int is_f32,
+                                  void* stream) {
+  if (T_ <= 0 || n_heads <= 0) return 0;
+  if (dim < 1 || half < 0 || 2 * half > dim || half > 4096) return -2;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const int* ps = static_cast<const int*>(positions);
+  const float* fr = static_cast<const float*>(inv_freq);
+  float *q = static_cast<float*>(q32), *k = static_cast<float*>(k32);
+  const bool vec = dim % 4 == 0 && half % 4 == 0 && stride % 4 == 0 && off_q % 4 == 0 && off_k % 4 == 0 &&
+                   (reinterpret_cast<uintptr_t>(y) & (is_f32 ? 15 : 7)) == 0 && ((reinterpret_cast<uintptr_t>(q32) | reinterpret_cast<uintptr_t>(k32)) & 15) == 0;
+  const size_t lds = 2 * sizeof(float) * std::max(half, 1);
+#define BCG_RET(TYPE, VEC)                                                                                                        \
+  retention_prepare_kernel<TYPE, VEC><<<T_, NT, lds, s>>>(static_cast<const TYPE*>(y), stride, off_q, off_k, n_heads, dim, ps, fr, \
+                                                          half, amp, k_scale, q, k)
+  if (vec) BCG_BY_TYPE((BCG_RET(float, true)), (BCG_RET(bf16_t, true)));
+  else BCG_BY_TYPE((BCG_RET(float, false)), (BCG_RET(bf16_t, false)));
+#undef BCG_RET
+  return BCG_CHECK_LAUNCH();
+}
+
 BCG_API int bcg_delta_prepare(const void* c, int64_t c_stride, const void* y, int64_t y_stride, int off_beta, const void* a,
                               int64_t a_stride, int gd, const void* a_log, const void* dt_bias, void* q32, void* k32, void* g32,
                               void* beta, int T_, int H, int G, int dim, int is_f32, void* stream) {
@@ -908,7 +1039,7 @@ BCG_API int bcg_delta_prepare(const void* c, int64_t c_stride, const void* y, in
 
 BCG_API int bcg_gated_state_scan(const void* q32, const void* k32, const void* g32, const void* v, int64_t v_stride,
                                  const void* beta, const void* positions, const void* q_start, const void* state_rows,
-                                 void* state, int n_rows, void* out, int B, int H, int Gq, int dim, int vdim, int gd, int delta,
+                                 void* state, int n_rows, void* out, int B, int H, int Gq, int dim, int vdim, int gd, int g_const, int delta,
                                  int unit_last, int is_f32, void* stream) {
   if (B <= 0) return 0;
   if (dim < 1 || dim > 256 || H <= 0 || Gq <= 0 || H % Gq || H > 65535 || (delta && beta == nullptr) || (gd != 1 && gd != dim)) return -2;
@@ -919,7 +1050,7 @@ BCG_API int bcg_gated_state_scan(const void* q32, const void* k32, const void* g
   a.positions = static_cast<const int*>(positions); a.q_start = static_cast<const int*>(q_start);
   a.state_rows = static_cast<const int*>(state_rows);
   a.state = static_cast<float*>(state); a.out = static_cast<float*>(out);
-  a.n_rows = n_rows; a.H = H; a.Gq = Gq; a.dim = dim; a.vdim = vdim; a.gd = gd;
+  a.n_rows = n_rows; a.H = H; a.Gq = Gq; a.dim = dim; a.vdim = vdim; a.gd = gd; a.g_token = g_const ? 0 : H * gd;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (delta) return is_f32 ? launch_scan<float, true>(a, B, s) : launch_scan<bf16_t, true>(a, B, s);
   return is_f32 ? launch_scan<float, false>(a, B, s) : launch_scan<bf16_t, false>(a, B, s);
