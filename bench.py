@@ -123,9 +123,9 @@ def parse(argv=None):
     ap.add_argument("--verbose", action="store_true")
     ap.add_argument("--families", default="",
                     help="with --family-compare: only these families and their kernel groups (comma-separated, of mofidra, "
-                         "padadra, mabivik, sitidra, sadodra, decoder; default: all)")
+                         "padadra, mabivik, sitidra, sadodra, vagozen, decoder; default: all)")
     ap.add_argument("--family-compare", action="store_true",
-                    help="instead of the headline workload: prefill / decode tokens/s of the Mofidra, Padadra, Mabivik, Sitidra and Sadodra families beside "
+                    help="instead of the headline workload: prefill / decode tokens/s of the Mofidra, Padadra, Mabivik, Sitidra, Sadodra and Vagozen families beside "
                          "the Qwen3-style decoder at equal layer sizes, and their hot kernels against the roofline "
                          "(one GPU, random weights; utils/family_bench.py)")
     return ap.parse_args(argv)

@@ -1011,10 +1011,10 @@ class VagozenConfig:
         layers = tuple(VagozenLayer(e["type"], cls._mixer(e["type"], e["mixer"]), cls._mlp(e.get("mlp"))) for e in c["layers"])
         loop = c.get("loop") or {}
         start, stop, times = int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1))
-        if not 0 <= start <= max(start, stop) <= len(layers) or times < 1:
+        if not 0 <= start <= stop <= len(layers) or times < 1:
             raise ValueError("Vagozen: loop span outside the layer list")
         return cls(name=name, hidden_size=int(c["width"]), vocab_size=int(c["vocab"]), layers=layers, loop_start=start,
-                   loop_stop=max(start, stop), loop_times=times, rms_eps=float(c["norm"]["eps"]),
+                   loop_stop=stop, loop_times=times, rms_eps=float(c["norm"]["eps"]),
                    logit_scale=float(c.get("logit_scale", 1.0)))
 
     def to_dict(self) -> dict:

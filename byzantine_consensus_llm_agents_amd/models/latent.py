@@ -6,7 +6,8 @@ attention runs in the latent: head h's query becomes ``[W_uk[h]^T q_h | rotated 
 softmax-weighted sum of c is expanded by ``W_uv[h]`` afterwards, so all heads read one KV head and
 nothing per head is cached.  Queries come from the input or through a normed latent of their own
 (``q_rank``); the sigmoid output gate, if there is one (``gated``), has one column per value feature or
-one per head (``head_gate``); the rotated part turns in halves or in neighbouring pairs (``rot_pairs``); a layer may read an earlier layer's cache (``kv_from``) with projections of its own.
+one per head (``head_gate``); the rotated part turns in halves or in neighbouring pairs
+(``rot_pairs``); a layer may read an earlier layer's cache (``kv_from``) with projections of its own.
 """
 
 import torch
@@ -21,9 +22,10 @@ def latent_shapes(m, W: int, q: str) -> dict:
         out.update({q + "dq": (m.q_rank, W), q + "dq.norm": (m.q_rank,), q + "uq": (m.q_width, m.q_rank)})
     else:
         out[q + "q"] = (m.q_width, W)
-    out.update({q + "uk": (m.heads * m.dim, m.kv_rank), q + "uv": (m.heads * m.vdim, m.kv_rank), q + "o": (W, m.heads * m.vdim)})
+    out.update({q + "uk": (m.heads * m.dim, m.kv_rank), q + "uv": (m.heads * m.vdim, m.kv_rank)})
     if m.gated:
         out[q + "g"] = (m.gate_width, W)
+    out[q + "o"] = (W, m.heads * m.vdim)
     if m.kv_from < 0:
         out.update({q + "dkv": (m.key_width, W), q + "dkv.norm": (m.kv_rank,)})
     return out

@@ -1,4 +1,4 @@
-"""Prefill / decode throughput of the Mofidra, Padadra, Mabivik, Sitidra and Sadodra families beside the Qwen3-style decoder
+"""Prefill / decode throughput of the Mofidra, Padadra, Mabivik, Sitidra, Sadodra and Vagozen families beside the Qwen3-style decoder
 at equal layer sizes (random weights, synthetic tokens), and the hot kernels against their
 rooflines.  ``bench.py --family-compare`` prints the result as one JSON line.
 
@@ -40,6 +40,17 @@ query / key and 128 value features per head, a 128-wide latent (a cached row of 
 head) and no window.  Its closest relatives are Mabivik (latent attention, post norms on an fp32
 stream), Padadra (windowed attention with whole-projection norms) and Mofidra (dense gelu).
 
+Vagozen at equal size: the same width, query / KV head counts and feed-forward width (clamped gated:
+three matrices); four layers (attention, retention, latent attention, retention) run as two passes of a
+loop over the last two, so six layer runs; ``vagozen_flat`` runs the four layers once.  The attention has
+128 query / key and 128 value features per head, pair rotary on 128 of them with ramped frequencies and a
+512-key window that keeps the first 16 keys; the retention half as many heads of 128 x 256 state; the
+latent attention Mabivik's sizes (128 + 64 query / key features, a 768-wide query latent, a cached row of
+192 features) without a window.  Feed-forwards: dense behind attention and latent attention, top-2 of 8
+experts of ff/4 behind retention.  Its closest relatives are Mabivik (latent attention, the same scan, gated
+experts, post norms on an fp32 stream), Padadra (pair rotary, windowed attention), Sadodra (gated dense
+feed-forward, residual kernel with the row in registers).
+
 Rooflines: 2.5 PFLOP/s dense bf16 MFMA, 8 TB/s HBM.  A kernel's ``roof_frac`` is
 max(flops / peak, bytes / bandwidth) / measured time.  The recurrence runs on the vector ALUs:
 its compute roof is 157 TFLOP/s fp32.
@@ -50,15 +61,16 @@ import time
 
 import torch
 
-from ..models.config import MabivikConfig, MofidraConfig, ModelConfig, PadadraConfig, SadodraConfig, SitidraConfig
+from ..models.config import MabivikConfig, MofidraConfig, ModelConfig, PadadraConfig, SadodraConfig, SitidraConfig, VagozenConfig
 from ..models.mabivik import MabivikModel
 from ..models.mofidra import MofidraModel
 from ..models.padadra import PadadraModel
 from ..models.sadodra import SadodraModel
 from ..models.sitidra import SitidraModel
 from ..models.transformer import AttnMeta, DecoderModel
+from ..models.vagozen import VagozenModel
 from ..ops import get_ops
-from ..ops.reference import alibi_slopes
+from ..ops.reference import alibi_slopes, ramp_inv_freq
 
 PEAK_FLOPS, PEAK_BW = 2.5e15, 8.0e12
 PEAK_VALU = 157e12
@@ -138,6 +150,24 @@ def sadodra_config(s) -> SadodraConfig:
         layers.append({"type": "attention" if i % 2 == 0 else "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": s["ff"]}})
     return SadodraConfig.from_dict({"architecture": "Sadodra", "width": W, "vocab": s["vocab"], "max_positions": 8192,
                                     "norm": {"eps": 1e-5}, "layers": layers}, "sadodra-bench")
+
+
+def vagozen_config(s, loop: bool = True) -> VagozenConfig:
+    H, G, W = s["heads"], s["kv_heads"], s["width"]
+    att = {"heads": H, "kv_heads": G, "dim": 128, "vdim": 128, "scale": 0.088, "mask": {"size": 512, "keep_first": 16},
+           "rot": {"dims": 128, "base": 1e6, "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+    ret = {"heads": H // 2, "dim": 128, "vdim": 256, "decay": [1.0 - 2.0 ** (-5 - i % 8) for i in range(H // 2)],
+           "rot": {"dims": 128, "base": 1e6}}
+    lat = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 768, "kv_rank": 128, "scale": 0.072,
+           "rot": {"dims": 64, "base": 1e6}}
+    dense = {"kind": "dense", "ff": s["ff"], "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": s["ff"] // 4, "limit": 7.0}, "router": {"experts": 8, "top": 2}}
+    kinds = [("attention", att, dense), ("retention", ret, moe), ("latent_attention", lat, dense), ("retention", ret, moe)]
+    layers = [dict(zip(("type", "mixer", "mlp"), kinds[i % 4])) for i in range(s["layers"])]
+    c = {"architecture": "Vagozen", "width": W, "vocab": s["vocab"], "norm": {"eps": 1e-5}, "logit_scale": 0.5, "layers": layers}
+    if loop:
+        c["loop"] = {"start": s["layers"] - 2, "stop": s["layers"], "times": 2}
+    return VagozenConfig.from_dict(c, "vagozen-bench")
 
 
 def decoder_config(s) -> ModelConfig:
@@ -734,6 +764,137 @@ def biased_kernels(s, dev):
     return out
 
 
+def retention_kernels(s, dev):
+    """Vagozen's kernels beside the like kernels of Mabivik, Padadra, Sadodra and Mofidra at the same shapes."""
+    ops = get_ops("hip")
+    H, G, W, ff = s["heads"], s["kv_heads"], s["width"], s["ff"]
+    bf = torch.bfloat16
+    out = {}
+    n, ctx, window, keep = 8, 1024, 512, 16
+    T, b = n * ctx, 64
+    meta, nb = step_meta(n, ctx, ctx, 64, dev, True)
+    dmeta, nbd = step_meta(b, ctx, 1, 64, dev, True)
+    nb = max(nb, nbd)
+    pairs_w = sum(min(i + 1, window) for i in range(ctx)) * n
+    pairs_k = sum(min(i + 1, window) + min(keep, max(0, i + 1 - window)) for i in range(ctx)) * n
+    pairs = ctx * (ctx + 1) // 2 * n
+    sink = torch.randn(H, device=dev)
+
+    def entry(name, **fracs):
+        out[name] = {}
+        for family, (t, flops, io, *peak) in fracs.items():
+            out[name][family + "_ms"] = round(t * 1e3, 4)
+            out[name][family + "_roof_frac"] = round(max(flops / (peak[0] if peak else PEAK_FLOPS), io / PEAK_BW) / t, 4)
+    # ---- windowed attention: kept first keys against a sink ----
+    kc, vc = torch.randn(nb, G, BS, 128, device=dev, dtype=bf), torch.randn(nb, G, 128, BS, device=dev, dtype=bf)
+    for name, rows, m_, timer in (("prefill_attention", T, meta, _time), ("decode_attention", b, dmeta, _graph_time)):
+        q = torch.randn(rows, H, 128, device=dev, dtype=bf)
+        args = (m_, 0.088, 1, 0.0, -1.0, 1.0, 128, window)
+        io = T * (H + G) * 256 * 2
+        entry(name, vagozen=(timer(lambda: ops.multimap_attention(q, kc, vc, *args, keep=keep)), 2 * H * 256 * (pairs_k if rows == T else b * (window + keep)),
+                             io if rows == T else b * (window + keep) * G * 256 * 2),
+              padadra=(timer(lambda: ops.multimap_attention(q, kc, vc, *args, sink)), 2 * H * 256 * (pairs_w if rows == T else b * window),
+                       io if rows == T else b * window * G * 256 * 2))
+    # ---- latent attention: one kernel; all keys against a window ----
+    for name, rows, m_, timer in (("prefill_latent_attention", T, meta, _time), ("decode_latent_attention", b, dmeta, _graph_time)):
+        res = {}
+        q = torch.randn(rows, H, 192, device=dev, dtype=bf)
+        kl, vl = torch.randn(nb, 1, BS, 192, device=dev, dtype=bf), torch.randn(nb, 1, 128, BS, device=dev, dtype=bf)
+        for family, win in (("vagozen", 0), ("mabivik", window)):
+            np_ = (pairs_w if win else pairs) if rows == T else b * (win or ctx)
+            io = T * (H + 1) * 320 * 2 if rows == T else b * (win or ctx) * 320 * 2
+            res[family] = (timer(lambda: ops.multimap_attention(q, kl, vl, m_, 0.072, 1, 0.0, -1.0, 1.0, 128, win, None)), 2 * H * 320 * np_, io)
+        entry(name, **res)
+    # ---- residual update + next norm: two RMS norms, and with the entry of a pass ----
+    w1, b1, w2, b2 = (torch.randn(W, device=dev) for _ in range(4))
+    table = torch.randn(s["vocab"], W, device=dev, dtype=bf)
+    for rows, timer in ((T, _time), (b, _graph_time)):
+        x32, a, p32 = torch.randn(rows, W, device=dev), torch.randn(rows, W, device=dev, dtype=bf), torch.randn(rows, W, device=dev)
+        tok = torch.randint(0, s["vocab"], (rows,), dtype=torch.int32, device=dev)
+        io = rows * W * (4 + 4 + 2 + 2)
+        it = dict(iters=20) if rows == T else dict(iters=50)
+        entry(f"residual_norm_{rows}_rows",
+              vagozen=(timer(lambda: ops.residual_post_norm(x32, a, ("rms", w1, 1e-5), ("rms", w2, 1e-5), bf), **it), 0, io),
+              sadodra=(timer(lambda: ops.residual_post_norm(x32, a, ("ln", w1, b1, 1e-5), ("copy",), bf), **it), 0, io),
+              mabivik=(timer(lambda: ops.residual_post_norm(x32, a, ("dyt", 0.5, w1, b1), ("dyt", 0.7, w2, b2), bf), **it), 0, io),
+              mofidra=(timer(lambda: ops.residual_add_rmsnorm32(x32, [a], w1, 1e-5, 1.0, bf), **it), 0, io))
+        entry(f"residual_norm_fp32_part_{rows}_rows",
+              vagozen=(timer(lambda: ops.residual_post_norm(x32, p32, ("rms", w1, 1e-5), ("rms", w2, 1e-5), bf), **it), 0, io + rows * W * 2),
+              mabivik=(timer(lambda: ops.residual_post_norm(x32, p32, ("rms", w1, 1e-5), ("dyt", 0.7, w2, b2), bf), **it), 0, io + rows * W * 2))
+        entry(f"residual_norm_pass_entry_{rows}_rows",
+              vagozen=(timer(lambda: ops.residual_post_norm(x32, a, ("rms", w1, 1e-5), ("rms", w2, 1e-5), bf, (w1, tok, table)), **it), 0, io + rows * W * 2))
+    tok = torch.randint(0, s["vocab"], (T,), dtype=torch.int32, device=dev)
+    entry("embedding", vagozen=(_time(lambda: ops.embed_scale_rmsnorm(tok, table, 1.0, w1, 1e-5, 0.0, bf, w2), iters=20), 0, T * W * (2 + 4 + 2)),
+          mofidra=(_time(lambda: ops.embed_scale_rmsnorm(tok, table, 1.0, w1, 1e-5, 1.0, bf), iters=20), 0, T * W * (2 + 4 + 2)))
+    # ---- cache writes ----
+    width = (H + 2 * G) * 128
+    qn, kn, inv = torch.ones(H * 128, device=dev), torch.ones(G * 128, device=dev), torch.rand(64, device=dev)
+    for name, rows, m_ in (("cache_write", T, meta), ("cache_write_decode", b, dmeta)):
+        y = torch.randn(rows, width, device=dev, dtype=bf)
+        io = rows * width * 2 * 2
+        entry(name, vagozen=(_graph_time(lambda: ops.rope_pairs_kv_write(y, m_.positions, m_.slots, H, G, 128, 128, None, None, 1e-5, inv, None, kc, vc,
+                                                                         amp=1.1), iters=50), 0, io),
+              padadra=(_graph_time(lambda: ops.rope_pairs_kv_write(y, m_.positions, m_.slots, H, G, 128, 128, qn, kn, 1e-5, inv[:32].contiguous(), inv, kc, vc),
+                                   iters=50), 0, io))
+        yl = torch.randn(rows, 768 + 192, device=dev, dtype=bf)
+        kl, vl = torch.randn(nb, 1, BS, 192, device=dev, dtype=bf), torch.randn(nb, 1, 128, BS, device=dev, dtype=bf)
+        qs, qd = torch.randn(rows, H, 192, device=dev, dtype=bf), torch.empty(rows, H, 192, device=dev, dtype=bf)
+        fr = inv[:32].contiguous()
+        res, res2 = {}, {}
+        for family, pr in (("vagozen", True), ("mabivik", False)):
+            res[family] = (_graph_time(lambda: ops.latent_kv_write(yl, 768, 128, 64, qn[:128], 1e-5, m_.positions, m_.slots, fr, 1.0, kl, vl, pr), iters=50),
+                           0, rows * (2 * 192 + 128) * 2)
+            res2[family] = (_graph_time(lambda: ops.rope_tail(qs, 128, qd, 128, m_.positions, fr, 1.0, pr), iters=50), 0, rows * H * 64 * 4)
+        entry("latent_" + name, **res)
+        entry("query_tail_rotary" + name[len("cache_write"):], **res2)
+    # ---- activations ----
+    for rows, timer in ((T, _time), (b, _graph_time)):
+        both = torch.randn(rows, 2 * ff, device=dev, dtype=bf)
+        entry(f"activation_{rows}_rows", vagozen=(timer(lambda: ops.gated_act(both, "clamped_glu", 7.0)), 0, rows * ff * 6),
+              sadodra=(timer(lambda: ops.gated_act(both, "gelu_tanh")), 0, rows * ff * 6))
+    # ---- routed experts ----
+    E, top, fe = 8, 2, ff // 4
+    for name, rows in (("prefill", T), ("decode", b)):
+        h = torch.randn(rows, W, device=dev, dtype=bf)
+        up, down = torch.randn(E, 2 * fe, W, device=dev, dtype=bf) * 0.02, torch.randn(E, W, fe, device=dev, dtype=bf) * 0.02
+        idx = torch.randint(0, E, (rows, 1), device=dev, dtype=torch.int32)
+        idx = torch.cat([idx, (idx + 1 + torch.randint(0, E - 1, (rows, 1), device=dev, dtype=torch.int32)) % E], 1).contiguous()
+        wts = torch.full((rows, top), 0.5, device=dev)
+        flops, io = 2 * 3 * rows * top * fe * W, 3 * E * fe * W * 2 + rows * W * 2 * (2 + 2 * top)
+        entry(f"experts_{name}", vagozen=(_time(lambda: ops.moe_experts(h, up, down, idx, wts, "clamped_glu", 7.0), iters=20), flops, io),
+              mabivik=(_time(lambda: ops.moe_experts(h, up, down, idx, wts, "silu_gated"), iters=20), flops, io))
+        rw, rb = torch.randn(E, W, device=dev) * 0.05, torch.randn(E, device=dev) * 0.1
+        entry(f"router_{name}", vagozen=(_time(lambda: ops.moe_route(h, rw, rb, 2), iters=20), 2 * rows * E * W, rows * W * 2))
+    # ---- retention: vectors, the recurrence, the output norm ----
+    Hr, d, vd = H // 2, 128, 256
+    decay = torch.rand(Hr, device=dev) * 0.1 + 0.9
+    for name, rows, m_ in (("prefill", T, meta), ("decode", b, dmeta)):
+        nseq = m_.q_start.numel() - 1
+        timer = (lambda f: _time(f, iters=10)) if name == "prefill" else (lambda f: _graph_time(f, iters=50))
+        y = torch.randn(rows, 2 * Hr * d + 2 * Hr * vd, device=dev, dtype=bf)
+        entry(f"retention_vectors_{name}",
+              vagozen=(timer(lambda: ops.retention_prepare(y, 0, Hr * d, Hr, d, d ** -0.5, m_.positions, inv, 1.0)), 0, rows * 2 * Hr * d * (2 + 4)))
+        q32, k32 = ops.retention_prepare(y, 0, Hr * d, Hr, d, d ** -0.5, m_.positions, inv, 1.0)
+        v = y[:, 2 * Hr * d:2 * Hr * d + Hr * vd]
+        S = torch.zeros(max(n, b) + 1, Hr, d, vd, device=dev)
+        flops = rows * Hr * d * vd * 6
+        io = rows * (2 * Hr * d * 4 + Hr * vd * (2 + 4)) + nseq * Hr * d * vd * 4 * 2
+        res = {"vagozen": (timer(lambda: ops.gated_state_scan(q32, k32, decay, v, None, m_, S, False)), flops, io, PEAK_VALU)}
+        qs, ks = torch.randn(rows, 2, 128, device=dev) * 0.1, torch.randn(rows, 2, 128, device=dev) * 0.1
+        gs, dts = torch.rand(rows, H, 1, device=dev), torch.rand(rows, H, device=dev)
+        vs = torch.randn(rows, H * 128, device=dev, dtype=bf)
+        Ss = torch.zeros(max(n, b) + 1, H, 128, 128, device=dev)
+        io2 = rows * (2 * 2 * 128 * 4 + H * 8 + H * 128 * 6) + nseq * H * 128 * 128 * 4 * 2
+        res["mabivik"] = (timer(lambda: ops.gated_state_scan(qs, ks, gs, vs, dts, m_, Ss, False)), rows * H * 128 * 128 * 6, io2, PEAK_VALU)
+        entry(f"retention_scan_{name}", **res)
+        del S, Ss
+        o32, z = torch.randn(rows, Hr, vd, device=dev), torch.randn(rows, Hr * vd, device=dev, dtype=bf)
+        o33, z3, wh = torch.randn(rows, H, 128, device=dev), torch.randn(rows, H * 128, device=dev, dtype=bf), torch.randn(128, device=dev)
+        entry(f"recurrent_out_norm_{name}", vagozen=(timer(lambda: ops.head_norm_gate(o32, None, 1e-5, z, bf, "silu")), 0, rows * Hr * vd * 8),
+              mabivik=(timer(lambda: ops.head_norm_gate(o33, wh, 1e-5, z3, bf, "silu")), 0, rows * H * 128 * 8))
+    return out
+
+
 def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
     dev = torch.device("cuda", torch.cuda.current_device())
     ops = get_ops("hip")
@@ -749,6 +910,8 @@ def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
                                  ("mabivik", lambda: MabivikModel(mabivik_config(s), ops, dev)),
                                  ("sitidra", lambda: SitidraModel(sitidra_config(s), ops, dev)),
                                  ("sadodra", lambda: SadodraModel(sadodra_config(s), ops, dev)),
+                                 ("vagozen", lambda: VagozenModel(vagozen_config(s), ops, dev)),
+                                 ("vagozen_flat", lambda: VagozenModel(vagozen_config(s, False), ops, dev)),
                                  ("decoder", lambda: DecoderModel(decoder_config(s), ops, dev))):
                 if families and label.split("_")[0] not in families:
                     continue
@@ -759,7 +922,7 @@ def run(sizes=("w2048", "w4096"), kernels=True, families=None) -> dict:
                 torch.cuda.empty_cache()
             groups = (("mofidra", "kernels", kernel_pairs), ("padadra", "state_kernels", state_kernels),
                       ("mabivik", "latent_kernels", latent_kernels), ("sitidra", "hyper_kernels", hyper_kernels),
-                      ("sadodra", "biased_kernels", biased_kernels))
+                      ("sadodra", "biased_kernels", biased_kernels), ("vagozen", "retention_kernels", retention_kernels))
             for family, key, fn in groups if kernels else ():
                 if not families or family in families:
                     entry[key] = fn(s, dev)
