@@ -34,6 +34,8 @@ def _segments(meta, T):
 
 
 def seqstate_ops(lib):
+    min_chunked = lib.bcg_retention_min_len()
+
     def embed_hashed_bigram_norm(tokens, meta, prev, table, scale, bigram, hash_mul, eps, gains, out_dtype):
         T, W = tokens.numel(), table.shape[1]
         _req(tokens.dtype == torch.int32 and tokens.is_contiguous() and tokens.dim() == 1, "tokens int32 [T]")
@@ -207,9 +209,19 @@ def seqstate_ops(lib):
             _req(beta.dtype == torch.float32 and beta.is_contiguous() and beta.shape == (T, H), "beta fp32 [T, H]")
         B = _segments(meta, T)
         out = torch.empty(T, H, vdim, dtype=torch.float32, device=g.device)
+        # a fixed decay per head and plain writes: long segments run as chunks of matrix products, the
+        # short ones among them (single tokens beside portions) token by token
+        skip = 0
+        if g_const and beta is None and not delta and not unit_last and not meta.decode and T - B + 1 >= min_chunked:
+            skip = min_chunked
+            _check(lib.bcg_retention_chunks(_p(q), _p(k), _p(g), _p(v), v.stride(0), _p(meta.positions), _p(meta.q_start),
+                                            _p(meta.state_rows), _p(state), state.shape[0], _p(out), B, H, Gq, dim, vdim, _act(v),
+                                            _stream()), "retention_chunks")
+            if B == 1:
+                return out
         _check(lib.bcg_gated_state_scan(_p(q), _p(k), _p(g), _p(v), v.stride(0), _p(beta), _p(meta.positions),
                                         _p(meta.q_start), _p(meta.state_rows), _p(state), state.shape[0], _p(out), B, H, Gq, dim,
-                                        vdim, gd, int(g_const), int(bool(delta)), int(bool(unit_last)), _act(v), _stream()), "gated_state_scan")
+                                        vdim, gd, int(g_const), skip, int(bool(delta)), int(bool(unit_last)), _act(v), _stream()), "gated_state_scan")
         return out
 
     def head_norm_gate(o, w, eps, gate, out_dtype, gate_act="sigmoid", floor=None):

@@ -660,6 +660,7 @@ struct ScanArgs {
   float* state;                                     // [n_rows, H, dim, vdim]
   float* out;                                       // [T, H, vdim]
   int n_rows, H, Gq, dim, vdim, gd, g_token;        // g_token: elements of g per token, H gd or 0
+  int skip_len;                                     // > 0: segments of at least this length are another kernel's
 };
 
 template <int CTRL>
@@ -687,7 +688,7 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void state_scan_kernel(ScanArgs a)
   const int b = blockIdx.x, h = blockIdx.y, j = (blockIdx.z * SCAN_WAVES + (tid >> 6)) * 8 + col;
   const int t0 = a.q_start[b], t1 = a.q_start[b + 1];
   const int sr = a.state_rows[b];
-  if (t1 <= t0 || sr < 0 || sr >= a.n_rows) return;
+  if (t1 <= t0 || sr < 0 || sr >= a.n_rows || (a.skip_len > 0 && t1 - t0 >= a.skip_len)) return;
   const bool col_ok = j < a.vdim;
   const int gq = h / (a.H / a.Gq);
   const int dim = a.dim, vdim = a.vdim;
@@ -1039,7 +1040,7 @@ BCG_API int bcg_delta_prepare(const void* c, int64_t c_stride, const void* y, in
 
 BCG_API int bcg_gated_state_scan(const void* q32, const void* k32, const void* g32, const void* v, int64_t v_stride,
                                  const void* beta, const void* positions, const void* q_start, const void* state_rows,
-                                 void* state, int n_rows, void* out, int B, int H, int Gq, int dim, int vdim, int gd, int g_const, int delta,
+                                 void* state, int n_rows, void* out, int B, int H, int Gq, int dim, int vdim, int gd, int g_const, int skip_len, int delta,
                                  int unit_last, int is_f32, void* stream) {
   if (B <= 0) return 0;
   if (dim < 1 || dim > 256 || H <= 0 || Gq <= 0 || H % Gq || H > 65535 || (delta && beta == nullptr) || (gd != 1 && gd != dim)) return -2;
@@ -1051,6 +1052,7 @@ BCG_API int bcg_gated_state_scan(const void* q32, const void* k32, const void* g
   a.state_rows = static_cast<const int*>(state_rows);
   a.state = static_cast<float*>(state); a.out = static_cast<float*>(out);
   a.n_rows = n_rows; a.H = H; a.Gq = Gq; a.dim = dim; a.vdim = vdim; a.gd = gd; a.g_token = g_const ? 0 : H * gd;
+  a.skip_len = skip_len;
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (delta) return is_f32 ? launch_scan<float, true>(a, B, s) : launch_scan<bf16_t, true>(a, B, s);
   return is_f32 ? launch_scan<float, false>(a, B, s) : launch_scan<bf16_t, false>(a, B, s);

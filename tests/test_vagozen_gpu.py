@@ -183,6 +183,35 @@ def test_retention_vectors(ops, dtype, H, d, half, off, pad):
             torch.testing.assert_close(a.cpu(), b, atol=3e-4, rtol=3e-4)
 
 
+@pytest.mark.parametrize("H,Gq,dim,vdim", [(3, 3, 16, 12), (4, 2, 64, 64), (2, 2, 128, 256), (6, 3, 40, 70), (2, 1, 7, 5), (3, 3, 130, 66), (2, 2, 256, 33), (1, 1, 20, 128)])
+def test_fixed_decay_recurrence(ops, dtype, H, Gq, dim, vdim):
+    """Segments of every kind in one packed step (single tokens, shorter and longer than the chunked form
+    takes, exactly one chunk, one token past it, several), fresh and continued, over stale rows; decays of
+    0 and 1 among them; the values a column range of wider rows."""
+    g = torch.Generator().manual_seed(dim + vdim)
+    decay = torch.tensor([(0.97, 0.0, 1.0, 0.9995, 0.5, 0.9)[h % 6] for h in range(H)])
+    parts = [(5, 1), (0, 64), (9, 2), (0, 15), (3, 16), (40, 65), (0, 1), (7, 17), (100, 200), (0, 130)]
+    rows = [3, 0, 7, 1, 9, 2, 8, 5, 4, 6]
+    meta = C.segments(parts, rows)
+    T = sum(n for _, n in parts)
+    q, k = torch.randn(T, Gq, dim, generator=g), torch.randn(T, Gq, dim, generator=g) * dim ** -0.5
+    y = torch.randn(T, 3 + H * vdim + 2, generator=g).to(dtype)
+    S = torch.randn(12, H, dim, vdim, generator=g)
+    Sd = S.to(DEV)
+    want = ref.gated_state_scan(q, k, decay, y[:, 3:3 + H * vdim], None, meta, S, False)
+    dev = C.segments(parts, rows, DEV)
+    got = ops.gated_state_scan(q.to(DEV), k.to(DEV), decay.to(DEV), y.to(DEV)[:, 3:3 + H * vdim], None, dev, Sd, False)
+    torch.testing.assert_close(got.cpu(), want, atol=2e-4, rtol=2e-4)
+    torch.testing.assert_close(Sd.cpu(), S, atol=2e-4, rtol=2e-4)
+    one = C.segments([(0, 300)], [5], DEV)   # one long segment alone
+    S1 = torch.full((6, H, dim, vdim), 9.0)
+    S1d = S1.to(DEV)
+    want = ref.gated_state_scan(q[:300], k[:300], decay, y[:300, 3:3 + H * vdim], None, C.segments([(0, 300)], [5]), S1, False)
+    got = ops.gated_state_scan(q[:300].to(DEV), k[:300].to(DEV), decay.to(DEV), y.to(DEV)[:300, 3:3 + H * vdim], None, one, S1d, False)
+    torch.testing.assert_close(got.cpu(), want, atol=2e-4, rtol=2e-4)
+    torch.testing.assert_close(S1d.cpu(), S1, atol=2e-4, rtol=2e-4)
+
+
 @pytest.mark.parametrize("R,RD,half,off", [(24, 8, 4, 5), (64, 32, 16, 0), (30, 6, 2, 3), (7, 2, 1, 1)])
 def test_latent_rows_turned_in_pairs(ops, dtype, R, RD, half, off):
     g = torch.Generator().manual_seed(R)
