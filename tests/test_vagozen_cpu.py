@@ -88,7 +88,7 @@ def test_oracle_pieces_by_hand():
     assert runs == [(0, None), (1, 0), (2, None), (1, 1), (2, None), (3, None)]
 
 
-@pytest.mark.parametrize("dims,base,scaling", [(64, 50000.0, (4.0, 512, 32.0, 1.0)), (12, 3000.0, (3.0, 64, 8.0, 1.0)), (6, 100.0, (8.0, 16, 32.0, 0.5)),
+@pytest.mark.parametrize("dims,base,scaling", [(48, 20000.0, (6.0, 384, 24.0, 2.0)), (12, 3000.0, (3.0, 64, 8.0, 1.0)), (6, 100.0, (8.0, 16, 32.0, 0.5)),
                                                (2, 10.0, (2.0, 4096, 1.0, 64.0)), (16, 1e6, None)])
 def test_ramped_frequencies(dims, base, scaling):
     got, amp = ramp_inv_freq(dims, base, scaling)
